@@ -4,3 +4,4 @@ from .duvulix import DuvulixConfig
 from .gumodra import GumodraConfig
 from .sagedra import SagedraConfig
 from .nelutar import NelutarConfig
+from .pemalorn import PemalornConfig

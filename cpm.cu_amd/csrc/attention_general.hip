@@ -669,7 +669,10 @@ extern "C" const char* cpmcu_qkv_rotate_store(const void* qkv, long ld, int dtyp
 //     and rotation), so dv == dk;
 //   * with norm_after q and k heads are rotated first and then divided by their root mean square (times the
 //     weight, if one is given);
-//   * with interleaved the rotation pairs neighbouring features (2i, 2i + 1) instead of (i, i + rot_dims/2).
+//   * with interleaved the rotation pairs neighbouring features (2i, 2i + 1) instead of (i, i + rot_dims/2);
+//   * q_scale (a number a query head) multiplies the finished query head, before it is rounded;
+//   * v_inv_freq (dv/2 frequencies): value heads of their own are rotated as well, over all dv features, in the same
+//     layout of pairs and without a magnitude (head_output_kernel turns what the attention makes of them back).
 // The projection's rows may be float where the cache is bfloat16 (rows that a convolution wrote).
 template <typename IT, typename T>
 __global__ __launch_bounds__(64) void qkv_norm_rotate_store_kernel(
@@ -677,7 +680,8 @@ __global__ __launch_bounds__(64) void qkv_norm_rotate_store_kernel(
     int dv, int rot_dims, const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w, float eps,
     int values_from_keys, const int* __restrict__ positions, const int* __restrict__ tok_slot,
     const float* __restrict__ inv_freq, float mag, T* __restrict__ kpool, T* __restrict__ vpool, PagedView pv,
-    int pool_hdk, int pool_hdv, int norm_after, int interleaved) {
+    int pool_hdk, int pool_hdv, int norm_after, int interleaved, const float* __restrict__ q_scale,
+    const float* __restrict__ v_inv_freq) {
     __shared__ float hs[AG_MAX_HD];
     const long t = blockIdx.x;
     const int y = blockIdx.y, lane = threadIdx.x;
@@ -688,8 +692,14 @@ __global__ __launch_bounds__(64) void qkv_norm_rotate_store_kernel(
     const long col = is_q ? (long)h * dk : (is_k ? (long)(nh + h) * dk : (long)(nh + nkv) * dk + (long)h * dv);
     const IT* src = qkv + t * ld + col;
     const long prow = is_q ? 0 : paged_row(pv, tok_slot[t], pos);
-    if (!is_q && !is_k) {               // a value head of its own: copied as it is
+    if (!is_q && !is_k) {               // a value head of its own: copied as it is, or rotated
         T* vd = vpool + value_index(prow, h, nkv, pool_hdv);
+        if (v_inv_freq) {
+            for (int i = lane; i < dv; i += 64) hs[i] = to_f32(src[i]) + (bias ? bias[col + i] : 0.f);
+            __syncthreads();
+            rotate_run(hs, vd, dv, dv, pos, v_inv_freq, 1.0f, DST_VALUES, 0, lane, 64, interleaved);
+            return;
+        }
         for (int i = lane; i < dv; i += 64) vd[value_d_offset(i)] = from_f32<T>(to_f32(src[i]) + (bias ? bias[col + i] : 0.f));
         return;
     }
@@ -726,6 +736,10 @@ __global__ __launch_bounds__(64) void qkv_norm_rotate_store_kernel(
         const float r = 1.0f / sqrtf(wave_sum(ss) / (float)width + eps);
         for (int i = lane; i < width; i += 64) hs[i] = hs[i] * r * nw[i];
     }
+    if (is_q && q_scale) {
+        const float qs = q_scale[h];
+        for (int i = lane; i < width; i += 64) hs[i] *= qs;
+    }
     __syncthreads();
     if (is_q) rotate_run(hs, q_out + (t * nh + h) * dk, dk, rot_dims, pos, inv_freq, mag, DST_ROWS, 0, lane, 64, interleaved);
     else rotate_run(hs, kpool + key_index(prow, h, nkv, pool_hdk), dk, rot_dims, pos, inv_freq, mag, DST_KEYS, 0, lane, 64,
@@ -739,8 +753,9 @@ extern "C" const char* cpmcu_qkv_norm_rotate_store(const void* qkv, long ld, int
                                                    const float* inv_freq, float mag, void* kpool, void* vpool,
                                                    const int* page_table, int table_width, int page_size, int pool_hdk,
                                                    int pool_hdv, int write_kv, int norm_after, int interleaved, int in_dtype,
-                                                   hipStream_t stream) {
+                                                   const float* q_scale, const float* v_inv_freq, hipStream_t stream) {
     CPMCU_REQUIRE(n > 0 && nh > 0 && nkv > 0 && dk > 0 && dv > 0, "qkv_norm_rotate_store: empty shape");
+    CPMCU_REQUIRE(!v_inv_freq || (dv % 2 == 0 && !values_from_keys), "qkv_norm_rotate_store: rotated values have heads of their own of an even size (%d)", dv);
     CPMCU_REQUIRE(dk <= AG_MAX_HD && dv <= AG_MAX_HD, "qkv_norm_rotate_store: key size %d / value size %d (up to %d are taken)",
                   dk, dv, AG_MAX_HD);
     CPMCU_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dk && (rot_dims == 0 || inv_freq),
@@ -758,7 +773,8 @@ extern "C" const char* cpmcu_qkv_norm_rotate_store(const void* qkv, long ld, int
 #define LAUNCH(ITv, Tv)                                                                                              \
     qkv_norm_rotate_store_kernel<ITv, Tv><<<grid, 64, 0, stream>>>(                                                  \
         (const ITv*)qkv, ld, bias, (Tv*)q_out, nh, nkv, dk, dv, rot_dims, q_norm_w, k_norm_w, eps, values_from_keys, \
-        positions, tok_slot, inv_freq, mag, (Tv*)kpool, (Tv*)vpool, pv, pool_hdk, pool_hdv, norm_after, interleaved)
+        positions, tok_slot, inv_freq, mag, (Tv*)kpool, (Tv*)vpool, pv, pool_hdk, pool_hdv, norm_after, interleaved, \
+        q_scale, v_inv_freq)
     // dtype: the cache's and q_out's element type; in_dtype: the projection rows' (float rows may feed a bfloat16 cache)
     if (dtype == CPMCU_F32 && in_dtype == CPMCU_F32) LAUNCH(float, float);
     else if (dtype == CPMCU_BF16 && in_dtype == CPMCU_BF16) LAUNCH(bf16_t, bf16_t);
@@ -769,76 +785,149 @@ extern "C" const char* cpmcu_qkv_norm_rotate_store(const void* qkv, long ld, int
     return nullptr;
 }
 
-// Latent attention: from a row [q heads: nh * (dim + rot) | down: rank + rot | ...] in one launch
-//   * y < nh: head y's rotated query part goes, rotated, behind the `rank` latent features of its query row
-//     q_out[t, y, rank:rank + rot] (the latent features themselves come from a product over heads);
-//   * y == nh (layers that own the cache): the latent c = rmsnorm(down[:rank]) * norm_w in float, into the key
-//     pages (features 0..rank) and the value pages, and the shared key part down[rank:], rotated, into the key
-//     pages behind it.
+// Latent attention's steps between its products and its attention in one launch; which of them a call does depends on
+// what it is given (grid y: the first nh rows, if there is a query source, then one each for the others):
+//   * queries (qsrc): head y's rotated query part qsrc[t, y * (dim + rot) + dim ..] goes, rotated, behind the `rank`
+//     latent features of its query row q_out[t, y, rank:rank + rot] (the latent features themselves come from a product
+//     over heads);
+//   * cache (down, layers that own it): the latent c = rmsnorm(down[:rank]) * norm_w in float, into the key pages
+//     (features 0..rank) and the value pages, and the shared key part down[rank:], rotated, into the key pages behind it;
+//   * query latent (cq_src): cq_out = rmsnorm(cq_src[:q_rank]) * cq_norm_w in float, rows of their own.
 template <typename T>
-__global__ __launch_bounds__(256) void latent_store_kernel(const T* __restrict__ proj, long ld, T* __restrict__ q_out,
-                                                           int nh, int dim, int rot, int rank,
+__global__ __launch_bounds__(256) void latent_store_kernel(const T* __restrict__ qsrc, long ldq, const T* __restrict__ down_src,
+                                                           long ldd, const T* __restrict__ cq_src, long ldc,
+                                                           T* __restrict__ q_out, int nh, int dim, int rot, int rank,
                                                            const float* __restrict__ norm_w, float eps,
-                                                           const int* __restrict__ positions,
+                                                           T* __restrict__ cq_out, const float* __restrict__ cq_norm_w,
+                                                           int q_rank, const int* __restrict__ positions,
                                                            const int* __restrict__ tok_slot,
-                                                           const float* __restrict__ inv_freq, float mag,
+                                                           const float* __restrict__ inv_freq, float mag, int interleaved,
                                                            T* __restrict__ kpool, T* __restrict__ vpool, PagedView pv,
                                                            int pool_hdk, int pool_hdv) {
     __shared__ float red[17];
     const long t = blockIdx.x;
-    const int y = blockIdx.y;
+    int y = blockIdx.y;
     const int pos = positions[t];
     const int qw = dim + rot, dk = rank + rot;
-    if (y < nh) {
-        rotate_run(proj + t * ld + (long)y * qw + dim, q_out + (t * nh + y) * dk + rank, rot, rot, pos, inv_freq, mag,
-                   DST_ROWS, 0, (int)threadIdx.x, (int)blockDim.x);
-        return;
+    if (qsrc) {
+        if (y < nh) {
+            rotate_run(qsrc + t * ldq + (long)y * qw + dim, q_out + (t * nh + y) * dk + rank, rot, rot, pos, inv_freq, mag,
+                       DST_ROWS, 0, (int)threadIdx.x, (int)blockDim.x, interleaved);
+            return;
+        }
+        y -= nh;
     }
-    const T* down = proj + t * ld + (long)nh * qw;
+    const bool cache = down_src && y == 0;
+    const T* src = cache ? down_src + t * ldd : cq_src + t * ldc;
+    const int width = cache ? rank : q_rank;
     float ss = 0.f;
-    for (int c = threadIdx.x; c < rank; c += blockDim.x) {
-        const float v = to_f32(down[c]);
+    for (int c = threadIdx.x; c < width; c += blockDim.x) {
+        const float v = to_f32(src[c]);
         ss += v * v;
     }
     ss = block_sum(ss, red);
-    const float rs = 1.0f / sqrtf(ss / (float)rank + eps);
+    const float rs = 1.0f / sqrtf(ss / (float)width + eps);
+    if (!cache) {
+        for (int c = threadIdx.x; c < width; c += blockDim.x) cq_out[t * q_rank + c] = from_f32<T>(to_f32(src[c]) * rs * cq_norm_w[c]);
+        return;
+    }
     const long prow = paged_row(pv, tok_slot[t], pos);
     T* kd = kpool + key_index(prow, 0, 1, pool_hdk);
     T* vd = vpool + value_index(prow, 0, 1, pool_hdv);
     for (int c = threadIdx.x; c < rank; c += blockDim.x) {
-        const T v = from_f32<T>(to_f32(down[c]) * rs * norm_w[c]);
+        const T v = from_f32<T>(to_f32(src[c]) * rs * norm_w[c]);
         kd[key_d_offset(c)] = v;
         vd[value_d_offset(c)] = v;
     }
-    rotate_run(down + rank, kd, rot, rot, pos, inv_freq, mag, DST_KEYS, rank, (int)threadIdx.x, (int)blockDim.x);
+    rotate_run(src + rank, kd, rot, rot, pos, inv_freq, mag, DST_KEYS, rank, (int)threadIdx.x, (int)blockDim.x, interleaved);
 }
 
-extern "C" const char* cpmcu_latent_store(const void* proj, long ld, int dtype, void* q_out, int n, int nh, int dim,
-                                          int rot, int rank, const float* norm_w, float eps, const int* positions,
-                                          const int* tok_slot, const float* inv_freq, float mag, void* kpool,
-                                          void* vpool, const int* page_table, int table_width, int page_size,
-                                          int pool_hdk, int pool_hdv, int write_cache, hipStream_t stream) {
+extern "C" const char* cpmcu_latent_store(const void* qsrc, long ldq, const void* down, long ldd, const void* cq_src, long ldc,
+                                          int dtype, void* q_out, int n, int nh, int dim, int rot, int rank,
+                                          const float* norm_w, float eps, void* cq_out, const float* cq_norm_w, int q_rank,
+                                          const int* positions, const int* tok_slot, const float* inv_freq, float mag,
+                                          int interleaved, void* kpool, void* vpool, const int* page_table, int table_width,
+                                          int page_size, int pool_hdk, int pool_hdv, hipStream_t stream) {
     CPMCU_REQUIRE(n > 0 && nh > 0 && dim > 0 && rank > 0 && rot >= 0 && rot % 2 == 0, "latent_store: bad shape");
     CPMCU_REQUIRE(rot == 0 || inv_freq, "latent_store: frequencies missing");
-    CPMCU_REQUIRE(ld >= (long)nh * (dim + rot) + (write_cache ? rank + rot : 0), "latent_store: rows of %ld too short", ld);
-    CPMCU_REQUIRE(!write_cache || (norm_w && kpool && vpool && page_table && page_size % 32 == 0 && pool_hdk % 16 == 0 &&
-                                   pool_hdv % 16 == 0 && pool_hdk >= rank + rot && pool_hdv >= rank),
+    if (rot == 0) qsrc = nullptr;                 // nothing of the queries is rotated
+    if (!qsrc && !down && !cq_src) return nullptr;
+    CPMCU_REQUIRE(!qsrc || (q_out && ldq >= (long)nh * (dim + rot)), "latent_store: query rows of %ld too short", ldq);
+    CPMCU_REQUIRE(!down || ldd >= rank + rot, "latent_store: rows of %ld too short", ldd);
+    CPMCU_REQUIRE(!cq_src || (q_rank > 0 && cq_out && cq_norm_w && ldc >= q_rank), "latent_store: query latent of %d in rows of %ld", q_rank, ldc);
+    CPMCU_REQUIRE(!down || (norm_w && kpool && vpool && page_table && tok_slot && page_size % 32 == 0 && pool_hdk % 16 == 0 &&
+                            pool_hdv % 16 == 0 && pool_hdk >= rank + rot && pool_hdv >= rank),
                   "latent_store: the cache takes pages of a multiple of 32 tokens and head sizes in steps of 16");
-    CPMCU_REQUIRE(nh < 65535, "latent_store: %d heads exceed the launch grid", nh);
-    if (!write_cache && rot == 0) return nullptr;
+    CPMCU_REQUIRE(nh < 65534, "latent_store: %d heads exceed the launch grid", nh);
     PagedView pv{page_table, table_width, page_size};
-    dim3 grid(n, nh + (write_cache ? 1 : 0));
-    const int block = rank >= 256 ? 256 : 64;
-    if (dtype == CPMCU_F32)
-        latent_store_kernel<float><<<grid, block, 0, stream>>>((const float*)proj, ld, (float*)q_out, nh, dim, rot, rank,
-                                                               norm_w, eps, positions, tok_slot, inv_freq, mag,
-                                                               (float*)kpool, (float*)vpool, pv, pool_hdk, pool_hdv);
-    else if (dtype == CPMCU_BF16)
-        latent_store_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)proj, ld, (bf16_t*)q_out, nh, dim, rot, rank,
-                                                                norm_w, eps, positions, tok_slot, inv_freq, mag,
-                                                                (bf16_t*)kpool, (bf16_t*)vpool, pv, pool_hdk, pool_hdv);
-    else
-        CPMCU_FAIL("latent_store: unknown dtype %d", dtype);
+    dim3 grid(n, (qsrc ? nh : 0) + (down ? 1 : 0) + (cq_src ? 1 : 0));
+    const int block = ((down && rank >= 256) || (cq_src && q_rank >= 256)) ? 256 : 64;
+#define LAUNCH(T)                                                                                                     \
+    latent_store_kernel<T><<<grid, block, 0, stream>>>((const T*)qsrc, ldq, (const T*)down, ldd, (const T*)cq_src, ldc, \
+                                                       (T*)q_out, nh, dim, rot, rank, norm_w, eps, (T*)cq_out, cq_norm_w, \
+                                                       q_rank, positions, tok_slot, inv_freq, mag, interleaved,       \
+                                                       (T*)kpool, (T*)vpool, pv, pool_hdk, pool_hdv)
+    if (dtype == CPMCU_F32) LAUNCH(float);
+    else if (dtype == CPMCU_BF16) LAUNCH(bf16_t);
+    else CPMCU_FAIL("latent_store: unknown dtype %d", dtype);
+#undef LAUNCH
     CPMCU_LAUNCH_CHECK("latent_store");
+    return nullptr;
+}
+
+// What some designs put between attention and output projection, a workgroup a token: with inv_freq the values were
+// cached rotated by their own positions (over all dv features) and every head's sum is turned back by the query's
+// position (pairs (i, i + dv/2), or neighbours when interleaved); with gate the head is multiplied by
+// sigmoid(gate[t, head]), a number a head.  The cos and sin of a token's angles are formed once, for all its heads.
+template <typename IT, typename T>
+__global__ __launch_bounds__(256) void head_output_kernel(const IT* __restrict__ o, T* __restrict__ out, int nh, int dv,
+                                                          const int* __restrict__ positions,
+                                                          const float* __restrict__ inv_freq, int interleaved,
+                                                          const T* __restrict__ gate, long ldg) {
+    __shared__ float cs[AG_MAX_HD / 2], sn[AG_MAX_HD / 2];
+    const long t = blockIdx.x;
+    const int half = dv / 2;
+    const IT* src = o + t * nh * dv;
+    T* dst = out + t * nh * dv;
+    if (!inv_freq) {
+        for (int i = threadIdx.x; i < nh * dv; i += 256) {
+            float v = to_f32(src[i]);
+            if (gate) v /= 1.0f + expf(-to_f32(gate[t * ldg + i / dv]));
+            dst[i] = from_f32<T>(v);
+        }
+        return;
+    }
+    const float pos = (float)positions[t];
+    for (int i = threadIdx.x; i < half; i += 256) {
+        const float ang = pos * inv_freq[i];
+        cs[i] = cosf(ang);
+        sn[i] = sinf(ang);
+    }
+    __syncthreads();
+    for (int j = threadIdx.x; j < nh * half; j += 256) {
+        const int h = j / half, i = j - h * half;
+        const int ia = h * dv + (interleaved ? 2 * i : i), ib = h * dv + (interleaved ? 2 * i + 1 : i + half);
+        const float u = to_f32(src[ia]), v = to_f32(src[ib]);
+        const float g = gate ? 1.0f / (1.0f + expf(-to_f32(gate[t * ldg + h]))) : 1.0f;
+        dst[ia] = from_f32<T>(g * (u * cs[i] + v * sn[i]));
+        dst[ib] = from_f32<T>(g * (v * cs[i] - u * sn[i]));
+    }
+}
+
+extern "C" const char* cpmcu_head_output(const void* o, int o_dtype, void* out, int dtype, int n, int nh, int dv,
+                                         const int* positions, const float* inv_freq, int interleaved, const void* gate,
+                                         long ldg, hipStream_t stream) {
+    CPMCU_REQUIRE(n > 0 && nh > 0 && dv > 0 && dv <= AG_MAX_HD, "head_output: empty shape or heads of %d (up to %d)", dv, AG_MAX_HD);
+    CPMCU_REQUIRE(!inv_freq || (positions && dv % 2 == 0), "head_output: rotated values have an even size (%d)", dv);
+    CPMCU_REQUIRE(!gate || ldg >= nh, "head_output: gate rows of %ld for %d heads", ldg, nh);
+#define LAUNCH(IT, T)                                                                                              \
+    head_output_kernel<IT, T><<<n, 256, 0, stream>>>((const IT*)o, (T*)out, nh, dv, positions, inv_freq, interleaved, \
+                                                     (const T*)gate, ldg)
+    if (o_dtype == CPMCU_F32 && dtype == CPMCU_F32) LAUNCH(float, float);
+    else if (o_dtype == CPMCU_F32 && dtype == CPMCU_BF16) LAUNCH(float, bf16_t);
+    else if (o_dtype == CPMCU_BF16 && dtype == CPMCU_BF16) LAUNCH(bf16_t, bf16_t);
+    else CPMCU_FAIL("head_output: unsupported dtypes in=%d out=%d", o_dtype, dtype);
+#undef LAUNCH
+    CPMCU_LAUNCH_CHECK("head_output");
     return nullptr;
 }

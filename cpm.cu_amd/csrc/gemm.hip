@@ -81,13 +81,14 @@ extern "C" const char* cpmcu_gemm_nt_plain(const void* X, long ldx, const void* 
 // The same product head by head: Y[m, h, :] = X[m, h, :] . W[h]^T for H heads with a weight [N, K] each (W is
 // [H, N, K]); head h's run of a row starts at h * hsx (X) and h * hsy (Y), so inputs and outputs may be slices
 // of wider rows.  With `gate` the rows of head h are multiplied by sigmoid(gate[m * ldg + h]) (an output gate
-// of one number a head).  blockIdx.z is the head.
+// of one number a head), or, gate_wide, element by element with sigmoid(gate[m * ldg + h * N + n]).  blockIdx.z is
+// the head.
 // ---------------------------------------------------------------------------
 template <typename XT, typename WT, typename OT>
 __global__ __launch_bounds__(256) void gemm_heads_kernel(const XT* __restrict__ X, long ldx, long hsx,
                                                          const WT* __restrict__ W, OT* __restrict__ Y, long ldy,
-                                                         long hsy, const XT* __restrict__ gate, long ldg, int M, int N,
-                                                         int K) {
+                                                         long hsy, const XT* __restrict__ gate, long ldg,
+                                                         int gate_wide, int M, int N, int K) {
     __shared__ float xs[GT_BK][GT_BM + 1];
     __shared__ float ws[GT_BK][GT_BN + 1];
     const int tx = threadIdx.x % 16, ty = threadIdx.x / 16;
@@ -125,26 +126,28 @@ __global__ __launch_bounds__(256) void gemm_heads_kernel(const XT* __restrict__ 
         const int m = m0 + ty * 4 + i;
         if (m >= M) continue;
         float gs = 1.f;
-        if (gate) gs = 1.0f / (1.0f + expf(-to_f32(gate[(long)m * ldg + h])));
+        if (gate && !gate_wide) gs = 1.0f / (1.0f + expf(-to_f32(gate[(long)m * ldg + h])));
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx * 4 + j;
-            if (n < N) Y[(long)m * ldy + n] = from_f32<OT>(gs * acc[i][j]);
+            if (n >= N) continue;
+            if (gate_wide) gs = 1.0f / (1.0f + expf(-to_f32(gate[(long)m * ldg + (long)h * N + n])));
+            Y[(long)m * ldy + n] = from_f32<OT>(gs * acc[i][j]);
         }
     }
 }
 
 extern "C" const char* cpmcu_gemm_nt_heads(const void* X, long ldx, long hsx, const void* W, void* Y, long ldy, long hsy,
-                                           const void* gate, long ldg, int in_dtype, int out_dtype, int M, int H, int N,
-                                           int K, hipStream_t stream) {
+                                           const void* gate, long ldg, int gate_wide, int in_dtype, int out_dtype, int M,
+                                           int H, int N, int K, hipStream_t stream) {
     CPMCU_REQUIRE(M > 0 && H > 0 && N > 0 && K > 0, "gemm_heads: empty shape M=%d heads=%d N=%d K=%d", M, H, N, K);
-    CPMCU_REQUIRE(ldx >= (H - 1) * hsx + K && ldy >= (H - 1) * hsy + N && (!gate || ldg >= H),
+    CPMCU_REQUIRE(ldx >= (H - 1) * hsx + K && ldy >= (H - 1) * hsy + N && (!gate || ldg >= (gate_wide ? (long)H * N : H)),
                   "gemm_heads: rows of %ld / %ld elements cannot hold %d heads", ldx, ldy, H);
     dim3 grid((N + GT_BN - 1) / GT_BN, (M + GT_BM - 1) / GT_BM, H);
     CPMCU_REQUIRE(grid.y <= 65535 && H <= 65535, "gemm_heads: M=%d or heads=%d too large for one launch", M, H);
 #define LAUNCH(T, OT)                                                                                          \
     gemm_heads_kernel<T, T, OT><<<grid, 256, 0, stream>>>((const T*)X, ldx, hsx, (const T*)W, (OT*)Y, ldy, hsy, \
-                                                          (const T*)gate, ldg, M, N, K)
+                                                          (const T*)gate, ldg, gate && gate_wide, M, N, K)
     if (in_dtype == CPMCU_F32 && out_dtype == CPMCU_F32) LAUNCH(float, float);
     else if (in_dtype == CPMCU_BF16 && out_dtype == CPMCU_BF16) LAUNCH(bf16_t, bf16_t);
     else if (in_dtype == CPMCU_BF16 && out_dtype == CPMCU_F32) LAUNCH(bf16_t, float);
@@ -167,7 +170,7 @@ template <int WM>
 __global__ __launch_bounds__(256) void gemm_heads_mfma_kernel(const bf16_t* __restrict__ X, long ldx, long hsx,
                                                               const bf16_t* __restrict__ W, bf16_t* __restrict__ Y,
                                                               long ldy, long hsy, const bf16_t* __restrict__ gate,
-                                                              long ldg, int M, int N, int K) {
+                                                              long ldg, int gate_wide, int M, int N, int K) {
     const int wave = __builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));
     const int lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
     const int h = blockIdx.z;
@@ -207,33 +210,37 @@ __global__ __launch_bounds__(256) void gemm_heads_mfma_kernel(const bf16_t* __re
         const int m = m0 + 4 * g + i;
         if (m >= M) continue;
         float gs = 1.f;
-        if (gate) gs = 1.0f / (1.0f + expf(-to_f32(gate[(long)m * ldg + h])));
+        if (gate && !gate_wide) gs = 1.0f / (1.0f + expf(-to_f32(gate[(long)m * ldg + h])));
         bf16_t* yr = Y + (long)h * hsy + (long)m * ldy;
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
-            if (n0 + 16 * j + r < N) yr[n0 + 16 * j + r] = f32_to_bf16(gs * acc[j][i]);
+        for (int j = 0; j < 4; ++j) {
+            const int n = n0 + 16 * j + r;
+            if (n >= N) continue;
+            if (gate_wide) gs = 1.0f / (1.0f + expf(-to_f32(gate[(long)m * ldg + (long)h * N + n])));
+            yr[n] = f32_to_bf16(gs * acc[j][i]);
+        }
     }
 }
 
 extern "C" const char* cpmcu_gemm_nt_heads_mfma(const void* X, long ldx, long hsx, const void* W, void* Y, long ldy,
-                                                long hsy, const void* gate, long ldg, int M, int H, int N, int K,
-                                                hipStream_t stream) {
+                                                long hsy, const void* gate, long ldg, int gate_wide, int M, int H, int N,
+                                                int K, hipStream_t stream) {
     CPMCU_REQUIRE(M > 0 && H > 0 && N > 0 && K > 0, "gemm_heads_mfma: empty shape M=%d heads=%d N=%d K=%d", M, H, N, K);
     CPMCU_REQUIRE(K % 8 == 0 && ldx % 8 == 0 && hsx % 8 == 0 && ((uintptr_t)X % 16 == 0) && ((uintptr_t)W % 16 == 0),
                   "gemm_heads_mfma: K, the row stride and the head stride of X must be multiples of 8 elements and "
                   "the operands start on 16-byte borders (K=%d, %ld, %ld)", K, ldx, hsx);
-    CPMCU_REQUIRE(ldx >= (H - 1) * hsx + K && ldy >= (H - 1) * hsy + N && (!gate || ldg >= H),
+    CPMCU_REQUIRE(ldx >= (H - 1) * hsx + K && ldy >= (H - 1) * hsy + N && (!gate || ldg >= (gate_wide ? (long)H * N : H)),
                   "gemm_heads_mfma: rows of %ld / %ld elements cannot hold %d heads", ldx, ldy, H);
     CPMCU_REQUIRE(H <= 65535, "gemm_heads_mfma: %d heads exceed the launch grid", H);
     if (M <= 16) {
         dim3 grid((N + 255) / 256, 1, H);
         gemm_heads_mfma_kernel<1><<<grid, 256, 0, stream>>>((const bf16_t*)X, ldx, hsx, (const bf16_t*)W, (bf16_t*)Y, ldy,
-                                                            hsy, (const bf16_t*)gate, ldg, M, N, K);
+                                                            hsy, (const bf16_t*)gate, ldg, gate && gate_wide, M, N, K);
     } else {
         dim3 grid((N + 63) / 64, (M + 63) / 64, H);
         CPMCU_REQUIRE(grid.y <= 65535, "gemm_heads_mfma: M=%d too large for one launch", M);
         gemm_heads_mfma_kernel<4><<<grid, 256, 0, stream>>>((const bf16_t*)X, ldx, hsx, (const bf16_t*)W, (bf16_t*)Y, ldy,
-                                                            hsy, (const bf16_t*)gate, ldg, M, N, K);
+                                                            hsy, (const bf16_t*)gate, ldg, gate && gate_wide, M, N, K);
     }
     CPMCU_LAUNCH_CHECK("gemm_nt_heads_mfma");
     return nullptr;

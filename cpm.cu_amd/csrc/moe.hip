@@ -5,7 +5,9 @@
 //    choice scores c = s + correction; the experts form `n_groups` equal groups of neighbours, a group's score is
 //    its largest c, or the sum of its two largest (group_fn), and only experts of the `keep_groups` best groups may be
 //    chosen (n_groups = 1: any; the others' c count as -inf); the `top` largest c are chosen (ties: the lower index),
-//    their weights are s / (sum of the chosen s + 1e-20) * weight_scale.  With w_sg (float [H]) it also
+//    their weights are s / (sum of the chosen s + 1e-20) * weight_scale, or s * weight_scale without `normalize`.  The
+//    router may have more rows than there are experts with matrices: the rows behind those are identity experts,
+//    whose output is h_t itself; the kernels below skip them and the last one adds their share.  With w_sg (float [H]) it also
 //    gives sigmoid(w_sg . h), the gate of an expert that every token uses.
 //  * moe_gated_kernel: act[t, k, :] = act(Wg_e h_t) * (Wu_e h_t) for the k-th chosen expert e of token t (the
 //    nonlinearities of common.h: SiLU, or the clamped swish with its limit); the experts' gate and up rows are
@@ -85,7 +87,7 @@ __global__ __launch_bounds__(64) void moe_select_kernel(const float* __restrict_
                                                         const float* __restrict__ correction, int has_sg, int E,
                                                         int n_groups, int keep_groups, int top, int* __restrict__ idx_out,
                                                         float* __restrict__ w_out, float* __restrict__ sg_out,
-                                                        int score_fn, int group_fn, float weight_scale) {
+                                                        int score_fn, int group_fn, float weight_scale, int normalize) {
     __shared__ float z[MOE_MAX_EXPERTS];      // logits, then softmax scores
     __shared__ float c[MOE_MAX_EXPERTS];      // choice scores; -inf once an expert is chosen or shut out
     __shared__ float gs[MOE_MAX_EXPERTS];     // group scores
@@ -170,14 +172,14 @@ __global__ __launch_bounds__(64) void moe_select_kernel(const float* __restrict_
         }
         __builtin_amdgcn_wave_barrier();
     }
-    const float norm = weight_scale / (chosen_sum + 1e-20f);
+    const float norm = normalize ? weight_scale / (chosen_sum + 1e-20f) : weight_scale;
     for (int r = lane; r < top; r += 64) w_out[t * top + r] *= norm;
 }
 
 extern "C" const char* cpmcu_moe_route(const void* h, long ldh, int dtype, const float* wr, const float* correction,
                                        const float* w_sg, int n, int H, int E, int n_groups, int keep_groups, int top,
                                        float* logits, int* idx_out, float* w_out, float* sg_out, int score_fn,
-                                       int group_fn, float weight_scale, hipStream_t stream) {
+                                       int group_fn, float weight_scale, int normalize, hipStream_t stream) {
     CPMCU_REQUIRE((score_fn == MOE_SCORE_SOFTMAX || score_fn == MOE_SCORE_SIGMOID) &&
                   (group_fn == MOE_GROUP_MAX || group_fn == MOE_GROUP_TOP2_SUM),
                   "moe_route: unknown score function %d or group score %d", score_fn, group_fn);
@@ -197,7 +199,7 @@ extern "C" const char* cpmcu_moe_route(const void* h, long ldh, int dtype, const
         CPMCU_FAIL("moe_route: unknown dtype %d", dtype);
     CPMCU_LAUNCH_CHECK("moe_logits");
     moe_select_kernel<<<n, 64, 0, stream>>>(logits, correction, w_sg ? 1 : 0, E, n_groups, keep_groups, top, idx_out, w_out,
-                                            sg_out, score_fn, group_fn, weight_scale);
+                                            sg_out, score_fn, group_fn, weight_scale, normalize);
     CPMCU_LAUNCH_CHECK("moe_select");
     return nullptr;
 }
@@ -208,10 +210,11 @@ extern "C" const char* cpmcu_moe_route(const void* h, long ldh, int dtype, const
 template <typename T>
 __global__ __launch_bounds__(256) void moe_gated_kernel(const T* __restrict__ h, long ldh, const T* __restrict__ wgu,
                                                         const int* __restrict__ idx, T* __restrict__ act, int H, int F,
-                                                        int top, int act_fn, float act_limit) {
+                                                        int top, int E, int act_fn, float act_limit) {
     const long pair = blockIdx.x;
     const long t = pair / top;
     const int e = idx[pair];
+    if (e >= E) return;                 // an identity expert
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const T* hr = h + t * ldh;
     const T* wg = wgu + (long)e * 2 * F * H;
@@ -229,16 +232,17 @@ __global__ __launch_bounds__(256) void moe_gated_kernel(const T* __restrict__ h,
 }
 
 extern "C" const char* cpmcu_moe_gated(const void* h, long ldh, int dtype, const void* wgu, const int* idx, void* act,
-                                       int n, int H, int F, int top, int act_fn, float act_limit, hipStream_t stream) {
-    CPMCU_REQUIRE(n > 0 && H > 0 && F > 0 && top > 0, "moe_gated: empty shape");
+                                       int n, int H, int F, int top, int E, int act_fn, float act_limit,
+                                       hipStream_t stream) {
+    CPMCU_REQUIRE(n > 0 && H > 0 && F > 0 && top > 0 && E > 0, "moe_gated: empty shape");
     CPMCU_REQUIRE(CPMCU_ACT_KNOWN(act_fn), "moe_gated: unknown nonlinearity %d", act_fn);
     const int fy = (F + 4 * MOE_ROWS - 1) / (4 * MOE_ROWS);
     CPMCU_REQUIRE(fy <= 65535, "moe_gated: %d rows an expert exceed the launch grid", F);
     dim3 grid((unsigned)((long)n * top), fy);
     if (dtype == CPMCU_F32)
-        moe_gated_kernel<float><<<grid, 256, 0, stream>>>((const float*)h, ldh, (const float*)wgu, idx, (float*)act, H, F, top, act_fn, act_limit);
+        moe_gated_kernel<float><<<grid, 256, 0, stream>>>((const float*)h, ldh, (const float*)wgu, idx, (float*)act, H, F, top, E, act_fn, act_limit);
     else if (dtype == CPMCU_BF16)
-        moe_gated_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)h, ldh, (const bf16_t*)wgu, idx, (bf16_t*)act, H, F, top, act_fn, act_limit);
+        moe_gated_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)h, ldh, (const bf16_t*)wgu, idx, (bf16_t*)act, H, F, top, E, act_fn, act_limit);
     else
         CPMCU_FAIL("moe_gated: unknown dtype %d", dtype);
     CPMCU_LAUNCH_CHECK("moe_gated");
@@ -246,12 +250,13 @@ extern "C" const char* cpmcu_moe_gated(const void* h, long ldh, int dtype, const
 }
 
 // grid (tokens, ceil(H / 16)), 256 threads.  shared: the every-token expert's output [n, H] (or float partial
-// sums [parts][n][H]), multiplied by sg[t]; may be absent.
+// sums [parts][n][H]), multiplied by sg[t]; may be absent.  h: the experts' input, what identity experts (e >= E) add.
 template <typename T, typename ST>
 __global__ __launch_bounds__(256) void moe_down_kernel(const T* __restrict__ act, const T* __restrict__ wd,
                                                        const int* __restrict__ idx, const float* __restrict__ w,
                                                        const ST* __restrict__ shared, int shared_parts,
                                                        long shared_stride, const float* __restrict__ sg,
+                                                       const T* __restrict__ h, long ldh, int E,
                                                        float* __restrict__ out, int H, int F, int top) {
     const long t = blockIdx.x;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -261,13 +266,18 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const T* __restrict__ act
     for (int r = 0; r < MOE_ROWS; ++r) {
         const int c = c0 + r;
         if (c >= H) break;
-        float s = 0.f;
+        float s = 0.f, same = 0.f;
         for (int k = 0; k < top; ++k) {
             const int e = idx[t * top + k];
+            if (e >= E) {
+                same += w[t * top + k];
+                continue;
+            }
             s += w[t * top + k] * lane_dot<T, T>(wd + ((long)e * H + c) * F, act + (t * top + k) * F, F, lane, vec);
         }
         s = wave_sum(s);
         if (lane == 0) {
+            if (h && same != 0.f) s += same * to_f32(h[t * ldh + c]);
             if (shared) {
                 float v = 0.f;
                 for (int p = 0; p < shared_parts; ++p) v += to_f32(shared[(long)p * shared_stride + t * H + c]);
@@ -280,14 +290,15 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const T* __restrict__ act
 
 extern "C" const char* cpmcu_moe_down(const void* act, int dtype, const void* wd, const int* idx, const float* w,
                                       const void* shared, int shared_dtype, int shared_parts, long shared_stride,
-                                      const float* sg, float* out, int n, int H, int F, int top, hipStream_t stream) {
-    CPMCU_REQUIRE(n > 0 && H > 0 && F > 0 && top > 0, "moe_down: empty shape");
+                                      const float* sg, const void* h, long ldh, int E, float* out, int n, int H, int F,
+                                      int top, hipStream_t stream) {
+    CPMCU_REQUIRE(n > 0 && H > 0 && F > 0 && top > 0 && E > 0, "moe_down: empty shape");
     const int hy = (H + 4 * MOE_ROWS - 1) / (4 * MOE_ROWS);
     CPMCU_REQUIRE(hy <= 65535, "moe_down: a width of %d exceeds the launch grid", H);
     dim3 grid(n, hy);
 #define LAUNCH(Tv, STv)                                                                                            \
     moe_down_kernel<Tv, STv><<<grid, 256, 0, stream>>>((const Tv*)act, (const Tv*)wd, idx, w, (const STv*)shared,   \
-                                                       shared_parts, shared_stride, sg, out, H, F, top)
+                                                       shared_parts, shared_stride, sg, (const Tv*)h, ldh, E, out, H, F, top)
     const int sd = shared ? shared_dtype : CPMCU_F32;
     if (dtype == CPMCU_F32 && sd == CPMCU_F32) LAUNCH(float, float);
     else if (dtype == CPMCU_BF16 && sd == CPMCU_F32) LAUNCH(bf16_t, float);
@@ -310,7 +321,7 @@ extern "C" const char* cpmcu_moe_down(const void* act, int dtype, const void* wd
 //    features (two tiles of gate rows, two of up rows): 16 matrix instructions for 8 operand loads, operands
 //    straight from memory (the 4 wavefronts of a workgroup read the same rows of h, which meet in the CU's cache).
 //  * moe_down_mfma_kernel: y[pair] = Wd_e act[pair] (bf16); a wavefront owns the 64 rows and 64 columns.
-//  * moe_combine_kernel: out[t] = sum_k w[t, k] y[t, k] (+ sg[t] * shared[t]) in float, k in order.
+//  * moe_combine_kernel: out[t] = sum_k w[t, k] y[t, k] (h_t where the chosen expert is an identity expert) (+ sg[t] * shared[t]) in float, k in order.
 // ===========================================================================
 typedef __bf16 mbf16x8_t __attribute__((ext_vector_type(8)));
 typedef float mfloatx4_t __attribute__((ext_vector_type(4)));
@@ -325,7 +336,8 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int* __restrict__
     for (int e = threadIdx.x; e < E; e += 1024) counts[e] = 0;
     for (int i = threadIdx.x; i < max_tiles * MOE_TILE; i += 1024) rows[i] = -1;
     __syncthreads();
-    for (int p = threadIdx.x; p < n_pairs; p += 1024) atomicAdd(&counts[idx[p]], 1);
+    for (int p = threadIdx.x; p < n_pairs; p += 1024)
+        if (idx[p] < E) atomicAdd(&counts[idx[p]], 1);              // identity experts have no tiles
     __syncthreads();
     if (threadIdx.x == 0) {
         int t = 0;
@@ -342,6 +354,7 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int* __restrict__
     __syncthreads();
     for (int p = threadIdx.x; p < n_pairs; p += 1024) {
         const int e = idx[p];
+        if (e >= E) continue;
         rows[offs[e] + atomicAdd(&counts[e], 1)] = p;
     }
 }
@@ -476,12 +489,14 @@ template <typename ST>
 __global__ __launch_bounds__(256) void moe_combine_kernel(const bf16_t* __restrict__ y, const float* __restrict__ w,
                                                           const ST* __restrict__ shared, int shared_parts,
                                                           long shared_stride, const float* __restrict__ sg,
-                                                          float* __restrict__ out, long total, int H, int top) {
+                                                          const int* __restrict__ idx, const bf16_t* __restrict__ h, long ldh,
+                                                          int E, float* __restrict__ out, long total, int H, int top) {
     for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < total; i += (long)gridDim.x * 256) {
         const long t = i / H;
         const int c = (int)(i - t * H);
         float s = 0.f;
-        for (int k = 0; k < top; ++k) s += w[t * top + k] * to_f32(y[(t * top + k) * H + c]);
+        for (int k = 0; k < top; ++k)
+            s += w[t * top + k] * to_f32(idx[t * top + k] < E ? y[(t * top + k) * H + c] : h[t * ldh + c]);
         if (shared) {
             float v = 0.f;
             for (int p = 0; p < shared_parts; ++p) v += to_f32(shared[(long)p * shared_stride + i]);
@@ -519,10 +534,10 @@ extern "C" const char* cpmcu_moe_experts_mfma(const void* h, long ldh, const voi
     const int blocks = (int)((total + 255) / 256 < 8192 ? (total + 255) / 256 : 8192);
     if (!shared || shared_dtype == CPMCU_F32)
         moe_combine_kernel<float><<<blocks, 256, 0, stream>>>((const bf16_t*)y, w, (const float*)shared, shared_parts,
-                                                              shared_stride, sg, out, total, H, top);
+                                                              shared_stride, sg, idx, (const bf16_t*)h, ldh, E, out, total, H, top);
     else
         moe_combine_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)y, w, (const bf16_t*)shared, shared_parts,
-                                                               shared_stride, sg, out, total, H, top);
+                                                               shared_stride, sg, idx, (const bf16_t*)h, ldh, E, out, total, H, top);
     CPMCU_LAUNCH_CHECK("moe_combine");
     return nullptr;
 }

@@ -5,3 +5,4 @@ from . import duvulix
 from . import gumodra
 from . import sagedra
 from . import nelutar
+from . import pemalorn

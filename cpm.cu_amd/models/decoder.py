@@ -5,7 +5,8 @@ naming the layer to run and the cache entry it uses.  A layer may be named by
 several runs (its weights are shared; each run has a cache entry of its own
 unless it says otherwise), and a run may read the cache entry that an earlier
 run wrote instead of writing one (``writes_cache`` false): then the mixer only
-projects queries.  The model itself knows nothing about what the parts compute.
+projects queries.  A run may begin a pass over a span of layers whose input is
+made of the residual and of the embedding's output (``begins_pass``).  The model itself knows nothing about what the parts compute.
 
 Forward of a step (reference order: src/model/minicpm4/minicpm4_model.cuh:125-153):
 embedding -> runs of the schedule -> final norm on the wanted rows -> head.
@@ -21,6 +22,7 @@ from .. import ops
 from ..cache.paged import CacheNeeds
 from ..parts.base import Block, Norm, Part, ResidualStream, Runtime, StepContext, branch_for
 from ..parts.embedding import LMHead, TokenEmbedding
+from ..parts.loop_input import LoopInput
 
 
 @dataclass(frozen=True)
@@ -28,6 +30,7 @@ class Run:
     layer: int                    # index into DecoderModel.layers
     cache: int                    # cache entry this run uses
     writes_cache: bool = True     # False: read the entry another run wrote
+    begins_pass: Optional[int] = None     # the number of the pass that begins with this run (LoopInput)
 
 
 def sequential_schedule(n_layers: int) -> List[Run]:
@@ -36,15 +39,18 @@ def sequential_schedule(n_layers: int) -> List[Run]:
 
 class DecoderModel(Part):
     def __init__(self, config, embedding: TokenEmbedding, layers: Sequence[Block], final_norm: Norm, head: LMHead,
-                 schedule: Optional[Sequence[Run]] = None, streams: Optional[int] = None):
+                 schedule: Optional[Sequence[Run]] = None, streams: Optional[int] = None,
+                 loop_input: Optional[LoopInput] = None, shared: Sequence[Part] = ()):
         """``streams``: the residual is that many rows a token (hyper-connections), all equal to the embedding's
-        output at the start; the blocks mix them, and the last norm reads their sum."""
+        output at the start; the blocks mix them, and the last norm reads their sum.  ``loop_input``: what the runs
+        that begin a pass do first.  ``shared``: parts that several layers read and none owns (a table)."""
         self.config = config
         self.streams = int(streams) if streams else None
         self.embedding = embedding
         self.layers = list(layers)
         self.final_norm = final_norm
         self.head = head
+        self.loop_input, self.shared = loop_input, list(shared)
         self.schedule = list(schedule) if schedule is not None else sequential_schedule(len(self.layers))
         self._check_schedule()
 
@@ -53,6 +59,9 @@ class DecoderModel(Part):
         for r in self.schedule:
             if not 0 <= r.layer < len(self.layers):
                 raise ValueError(f"schedule names layer {r.layer}, the model has {len(self.layers)}")
+            if r.begins_pass is not None and (self.loop_input is None or self.streams
+                                              or not 0 <= r.begins_pass < self.loop_input.times):
+                raise ValueError(f"a run begins pass {r.begins_pass}, which the model's loop input does not have")
             if r.writes_cache:
                 if r.cache in written:
                     raise ValueError(f"cache entry {r.cache} is written by two runs of the schedule")
@@ -73,14 +82,15 @@ class DecoderModel(Part):
         return self.head.vocab_size
 
     def parts(self) -> List[Part]:
-        return [self.embedding] + self.layers + [self.final_norm, self.head]
+        return ([self.embedding] + self.shared + ([self.loop_input] if self.loop_input is not None else []) + self.layers
+                + [self.final_norm, self.head])
 
     def cache_needs(self) -> List[CacheNeeds]:
-        """What each cache entry needs: that of the mixer of the run that writes it."""
+        """What each cache entry needs: that of the block of the run that writes it."""
         needs: List[Optional[CacheNeeds]] = [None] * self.n_cache_entries
         for r in self.schedule:
             if r.writes_cache:
-                needs[r.cache] = self.layers[r.layer].mixer.cache_needs()
+                needs[r.cache] = self.layers[r.layer].cache_needs()
         if self.embedding_entry is not None:
             needs.append(self.embedding.cache_needs())
         return needs  # type: ignore[return-value]
@@ -96,8 +106,12 @@ class DecoderModel(Part):
                 lanes = ctx.ws.get("residual.streams", (self.streams,) + tuple(x.shape), torch.float32)
                 ops.streams_fill(x, lanes)
                 x = lanes
+            if self.loop_input is not None:
+                self.loop_input.start(x, ctx)
             stream = ResidualStream(x)
         for r in self.schedule:
+            if r.begins_pass is not None:
+                self.loop_input.forward(stream, ctx, r.begins_pass)
             self.layers[r.layer].forward(stream, ctx, ctx.cache.view(r.cache) if ctx.cache is not None else None,
                                          r.writes_cache)
         if ctx.logit_rows is None or ctx.logit_rows.numel() == 0:

@@ -687,13 +687,16 @@ def qkv_norm_rotate_store(qkv: torch.Tensor, q_out: torch.Tensor, nh: int, nkv: 
                           page_table: Optional[torch.Tensor], page_size: int, write_kv: bool = True,
                           bias: Optional[torch.Tensor] = None, q_norm: Optional[torch.Tensor] = None,
                           k_norm: Optional[torch.Tensor] = None, eps: float = 0.0, values_from_keys: bool = False,
-                          norm_after: bool = False, interleaved: bool = False):
+                          norm_after: bool = False, interleaved: bool = False, q_scale: Optional[torch.Tensor] = None,
+                          v_inv_freq: Optional[torch.Tensor] = None):
     """qkv_rotate_store with what some designs put between projection and rotation: ``bias`` (float32, as wide as
     a row of qkv) is added; q heads and k heads are divided by their root mean square (eps inside the root) and
     multiplied by a weight of dk numbers shared by the heads (q_norm, k_norm, float32 [dk]); with
     values_from_keys a row is [q | k] only and the value pages receive k as projected (with its bias, before norm
     and rotation).  With norm_after the q and k heads are rotated first and then divided by their root mean square
-    (times q_norm / k_norm where given, by nothing else where not).  ``interleaved`` as in qkv_rotate_store.  The
+    (times q_norm / k_norm where given, by nothing else where not).  ``interleaved`` as in qkv_rotate_store.
+    q_scale (float32 [nh]) multiplies a finished query head; v_inv_freq (float32 [dv/2]): value heads are rotated by
+    their positions as well, over all dv features (head_output turns what the attention makes of them back).  The
     rows of qkv may be float32 where q_out and the cache are bfloat16 (rows that a convolution wrote)."""
     ld = _ld(qkv, "qkv")
     n = qkv.shape[0]
@@ -715,6 +718,12 @@ def qkv_norm_rotate_store(qkv: torch.Tensor, q_out: torch.Tensor, nh: int, nkv: 
     for t, name in ((q_norm, "query norm weight"), (k_norm, "key norm weight")):
         if t is not None:
             _need(t, f"qkv {name}", torch.float32, (dk,))
+    if q_scale is not None:
+        _need(q_scale, "qkv query scales", torch.float32, (nh,))
+    if v_inv_freq is not None:
+        if dv % 2 or values_from_keys:
+            raise KernelError(f"qkv_norm_rotate_store: rotated values have heads of their own of an even size ({dv})")
+        _need(v_inv_freq, "qkv value inv_freq", torch.float32, (dv // 2,))
     tw = pk = pv = 0
     if write_kv:
         _need(tok_slot, "qkv token slots", torch.int32, (n,))
@@ -730,7 +739,7 @@ def qkv_norm_rotate_store(qkv: torch.Tensor, q_out: torch.Tensor, nh: int, nkv: 
         _p(tok_slot), _p(inv_freq), c_float(mag), _p(kpool if write_kv else None), _p(vpool if write_kv else None),
         _p(page_table if write_kv else None), c_int(tw), c_int(page_size), c_int(pk), c_int(pv),
         c_int(1 if write_kv else 0), c_int(1 if norm_after else 0), c_int(1 if interleaved else 0), c_int(_code(qkv)),
-        _stream()))
+        _p(q_scale), _p(v_inv_freq), _stream()))
 
 
 def _parts_of(t: torch.Tensor, n: int, H: int, name: str):
@@ -905,6 +914,136 @@ def streams_norm(x: torch.Tensor, branch: Optional[torch.Tensor], branch_bias: O
         _stream()))
 
 
+ROW_NORMS = {None: 0, "layer": 1, "rms": 2}
+
+
+def norm_rows(x: torch.Tensor, out: Optional[torch.Tensor], norm: Optional[str], weight: Optional[torch.Tensor] = None,
+              eps: float = 0.0, branch: Optional[torch.Tensor] = None, branch_scale: float = 1.0,
+              branch_bias: Optional[torch.Tensor] = None, branch_norm: Optional[torch.Tensor] = None,
+              branch_eps: float = 0.0, replace: bool = False, rows: Optional[torch.Tensor] = None,
+              convs: Sequence[torch.Tensor] = (), conv_state: Optional[torch.Tensor] = None,
+              slots: Optional[torch.Tensor] = None, out2: Optional[torch.Tensor] = None):
+    """One pass over the rows of the residual x (float32 [n, H]).  With a branch y = branch_scale * branch +
+    branch_bias ([n, H], or summed over the leading axis of [P, n, H]), divided by its root mean square and multiplied
+    by branch_norm where that is given; x += y, or x = y with ``replace`` (in place).  out (float32 or bfloat16
+    [n, H], may be columns of a wider tensor; None: only x is updated) = x, its layer norm without bias ('layer') or
+    its RMS norm ('rms') times weight.  With ``rows`` (int32 [R]) only those rows are computed, into out [R, H], and x
+    is left as it was.
+    convs (one or two, float32 [taps, H]), for steps in which every row is one sequence's only token: with h the normed
+    row, out = h + sum_j convs[0][j] h_(t-taps+1+j) and out2 likewise with convs[1]; the earlier rows come from
+    conv_state (float32 [slots, taps-1, H]) at slots[row], which moves on by one."""
+    _need(x, "rows residual", torch.float32, (None, None))
+    n, H = x.shape
+    if norm not in ROW_NORMS:
+        raise KernelError(f"norm_rows: norm '{norm}' ({sorted(k for k in ROW_NORMS if k)})")
+    if norm is not None:
+        _need(weight, "rows norm weight", torch.float32, (H,))
+    parts, stride, bcode = 1, 0, F32
+    if branch is not None:
+        parts, stride = _parts_of(branch, n, H, "rows branch")
+        bcode = _code(branch)
+        for t, name in ((branch_bias, "branch bias"), (branch_norm, "branch norm weight")):
+            if t is not None:
+                _need(t, f"rows {name}", torch.float32, (H,))
+    elif replace or branch_norm is not None or branch_bias is not None:
+        raise KernelError("norm_rows: a branch is missing")
+    n_out, ldo = n, H
+    if rows is not None:
+        _need(rows, "norm rows", torch.int32, (None,))
+        n_out = rows.shape[0]
+    if out is not None:
+        ldo = _ld(out, "rows out")
+        if tuple(out.shape) != (n_out, H):
+            raise KernelError(f"rows out: shape {tuple(out.shape)}, expected {(n_out, H)}")
+    elif branch is None or convs:
+        raise KernelError("norm_rows: nothing to write")
+    taps = 1
+    if convs:
+        if len(convs) > 2 or rows is not None:
+            raise KernelError("norm_rows: one or two convolutions over whole steps")
+        taps = convs[0].shape[0]
+        for w in convs:
+            _need(w, "rows convolution", torch.float32, (taps, H))
+        if taps > 1:
+            _need(conv_state, "rows convolution state", torch.float32, (None, taps - 1, H))
+            _need(slots, "rows slots", torch.int32, (n,))
+        if len(convs) == 2:
+            _need(out2, "rows second out", out.dtype, (n, H))
+            if ldo != H:
+                raise KernelError("norm_rows: two outputs are contiguous")
+    _check(_fn("rows", "cpmcu_norm_rows")(
+        _p(x), _p(branch), c_int(bcode), c_int(parts), c_long(stride), c_float(branch_scale), _p(branch_bias), _p(branch_norm),
+        c_float(branch_eps), c_int(1 if replace else 0), c_int(ROW_NORMS[norm]), _p(weight if norm is not None else None),
+        c_float(eps), _p(out), c_int(_code(out) if out is not None else F32), c_long(ldo), _p(rows), c_int(n_out), c_int(H),
+        _p(convs[0] if convs else None), _p(convs[1] if len(convs) > 1 else None), c_int(taps),
+        _p(conv_state if convs and taps > 1 else None), _p(slots if convs and taps > 1 else None),
+        _p(out2 if len(convs) > 1 else None), _stream()))
+
+
+def conv_rows(h: torch.Tensor, convs: Sequence[torch.Tensor], conv_state: Optional[torch.Tensor], outs: Sequence[torch.Tensor],
+              cu_q: torch.Tensor, seq_slot: torch.Tensor, max_q: int, update_state: bool = True):
+    """outs[k][t] = h[t] + sum_j convs[k][j] h[t-taps+1+j] over each sequence's tokens (one or two convolutions,
+    float32 [taps, H]); what lies before the step comes from conv_state (float32 [slots, taps-1, H], zeros at a
+    sequence's start), which moves on to the step's last rows.  cu_q int32 [B+1], seq_slot int32 [B]; max_q: the
+    longest run of tokens a sequence brings."""
+    _need(h, "convolution input", shape=(None, None))
+    n, H = h.shape
+    if not 1 <= len(convs) <= 2 or len(outs) != len(convs):
+        raise KernelError("conv_rows: one or two convolutions, an output each")
+    taps = convs[0].shape[0]
+    for w in convs:
+        _need(w, "rows convolution", torch.float32, (taps, H))
+    for o in outs:
+        _need(o, "convolution out", outs[0].dtype, (n, H))
+    if taps > 1:
+        _need(conv_state, "rows convolution state", torch.float32, (None, taps - 1, H))
+    _need(cu_q, "convolution sequence starts", torch.int32, (None,))
+    B = cu_q.shape[0] - 1
+    _need(seq_slot, "convolution sequence slots", torch.int32, (B,))
+    _check(_fn("rows", "cpmcu_conv_rows")(
+        _p(h), c_int(_code(h)), _p(convs[0]), _p(convs[1] if len(convs) > 1 else None), c_int(taps),
+        _p(conv_state if taps > 1 else None), _p(outs[0]), _p(outs[1] if len(outs) > 1 else None), c_int(_code(outs[0])),
+        _p(cu_q), _p(seq_slot), c_int(B), c_int(max_q), c_int(H), c_int(1 if update_state else 0), _stream()))
+
+
+def add_rows(x: torch.Tensor, a: Optional[torch.Tensor] = None, a_bias: Optional[torch.Tensor] = None,
+             f: Optional[torch.Tensor] = None, f_bias: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None):
+    """x += a + a_bias + f + f_bias in place (float32 [n, H]; a and f [n, H] or float partial sums [P, n, H], either may
+    be None), and out (float32 or bfloat16 [n, H], may be columns of a wider tensor) = x."""
+    _need(x, "rows residual", torch.float32, (None, None))
+    n, H = x.shape
+    ap, astr = _parts_of(a, n, H, "rows branch") if a is not None else (0, 0)
+    fp, fstr = _parts_of(f, n, H, "rows second branch") if f is not None else (0, 0)
+    for t, name in ((a_bias, "branch bias"), (f_bias, "second branch bias")):
+        if t is not None:
+            _need(t, f"rows {name}", torch.float32, (H,))
+    ldo = 0
+    if out is not None:
+        ldo = _ld(out, "rows out")
+        if tuple(out.shape) != (n, H):
+            raise KernelError(f"rows out: shape {tuple(out.shape)}, expected {(n, H)}")
+    _check(_fn("rows", "cpmcu_add_rows")(
+        _p(x), _p(a), c_int(_code(a) if a is not None else F32), c_int(ap), c_long(astr), _p(a_bias), _p(f),
+        c_int(_code(f) if f is not None else F32), c_int(fp), c_long(fstr), _p(f_bias), _p(out),
+        c_int(_code(out) if out is not None else F32), c_long(ldo), c_int(n), c_int(H), _stream()))
+
+
+def gated_lookup(z: torch.Tensor, table: torch.Tensor, offset: int, ids: torch.Tensor, out: torch.Tensor,
+                 activation: str = "gelu_tanh"):
+    """out[t, j] = act(z[t, j]) * table[ids[t], offset + j]; z [n, D] or float partial sums [P, n, D], table [V, W],
+    ids int32 [n], out [n, D] of the table's type; act SiLU or the tanh form of GELU."""
+    _need(out, "lookup out", shape=(None, None))
+    n, D = out.shape
+    parts, stride = _parts_of(z, n, D, "lookup gate")
+    _need(table, "lookup table", out.dtype, (None, None))
+    if offset < 0 or offset + D > table.shape[1]:
+        raise KernelError(f"gated_lookup: columns {offset}..{offset + D} of a table of {table.shape[1]}")
+    _need(ids, "lookup ids", torch.int32, (n,))
+    _check(_fn("rows", "cpmcu_gated_lookup")(_p(z), c_int(_code(z)), c_int(parts), c_long(stride), _p(table),
+                                             c_int(_code(table)), c_long(table.shape[1]), c_long(offset), _p(ids), _p(out),
+                                             c_int(n), c_int(D), c_int(GATE_ACTIVATIONS[activation]), _stream()))
+
+
 def pair_norm_mean(a: torch.Tensor, a_bias: Optional[torch.Tensor], b: torch.Tensor, b_bias: Optional[torch.Tensor],
                    wa: torch.Tensor, wb: torch.Tensor, eps: float, out: torch.Tensor):
     """out = (a / rms(a) * wa + b / rms(b) * wb) / 2 row by row in float, rms(v) = sqrt(mean(v^2) + eps): the
@@ -1068,13 +1207,13 @@ MOE_GROUP_SCORES = {"max": 0, "top2_sum": 1}
 def moe_route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.Tensor], shared_gate: Optional[torch.Tensor],
               n_groups: int, keep_groups: int, top: int, idx: torch.Tensor, weights: torch.Tensor,
               shared_out: Optional[torch.Tensor] = None, logits: Optional[torch.Tensor] = None,
-              score: str = "softmax", group_score: str = "max", weight_scale: float = 1.0):
+              score: str = "softmax", group_score: str = "max", weight_scale: float = 1.0, normalize: bool = True):
     """Routing of every token to ``top`` of E experts.  Logits router . h in float (router float32 [E, H]), scores
     s = softmax over the experts (``score`` 'sigmoid': of each logit alone); choice scores s + correction; the
     experts form n_groups equal groups of neighbours, of which only the keep_groups with the largest group score may
     be chosen from (``group_score`` 'max': a group's best choice score; 'top2_sum': the sum of its two best); the top
     largest choice scores win (ties: the lower index); weights = s of the chosen / (their sum + 1e-20) *
-    weight_scale.  idx int32 [n, top], weights float32 [n, top].
+    weight_scale (without ``normalize`` s * weight_scale).  idx int32 [n, top], weights float32 [n, top].
     shared_gate (float32 [H]): shared_out[t] = sigmoid(shared_gate . h[t]).  logits: float32 [n, E + 1] of scratch
     (allocated here when absent: a caller that must not allocate brings it)."""
     ldh = _ld(h, "router input")
@@ -1097,12 +1236,13 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.
     _check(_fn("moe", "cpmcu_moe_route")(_p(h), c_long(ldh), c_int(_code(h)), _p(router), _p(correction), _p(shared_gate),
                                          c_int(n), c_int(H), c_int(E), c_int(n_groups), c_int(keep_groups), c_int(top),
                                          _p(logits), _p(idx), _p(weights), _p(shared_out), c_int(MOE_SCORES[score]),
-                                         c_int(MOE_GROUP_SCORES[group_score]), c_float(weight_scale), _stream()))
+                                         c_int(MOE_GROUP_SCORES[group_score]), c_float(weight_scale), c_int(1 if normalize else 0), _stream()))
 
 
 def moe_gated(h: torch.Tensor, gate_up: torch.Tensor, idx: torch.Tensor, act: torch.Tensor, activation="silu"):
     """act[t, k] = act(Wg_e h[t]) * (Wu_e h[t]) for e = idx[t, k] (act: SiLU, or as gate_activation says); gate_up
-    [E, 2F, H] (an expert's gate rows, then its up rows), act [n, top, F], both of h's element type."""
+    [E, 2F, H] (an expert's gate rows, then its up rows), act [n, top, F], both of h's element type.  Pairs whose
+    expert is E or higher (identity experts, which have no matrices) are left out."""
     ldh = _ld(h, "experts input")
     n, H = h.shape
     _need(gate_up, "experts gate/up", h.dtype, (None, None, H))
@@ -1113,17 +1253,22 @@ def moe_gated(h: torch.Tensor, gate_up: torch.Tensor, idx: torch.Tensor, act: to
     top = idx.shape[1]
     _need(act, "experts act", h.dtype, (n, top, F2 // 2))
     _check(_fn("moe", "cpmcu_moe_gated")(_p(h), c_long(ldh), c_int(_code(h)), _p(gate_up), _p(idx), _p(act), c_int(n),
-                                         c_int(H), c_int(F2 // 2), c_int(top), *_act(activation), _stream()))
+                                         c_int(H), c_int(F2 // 2), c_int(top), c_int(E), *_act(activation), _stream()))
 
 
 def moe_down(act: torch.Tensor, down: torch.Tensor, idx: torch.Tensor, weights: torch.Tensor, out: torch.Tensor,
-             shared: Optional[torch.Tensor] = None, shared_gate: Optional[torch.Tensor] = None):
+             shared: Optional[torch.Tensor] = None, shared_gate: Optional[torch.Tensor] = None,
+             h: Optional[torch.Tensor] = None):
     """out[t] = sum_k weights[t, k] * Wd_e act[t, k] (+ shared_gate[t] * shared[t]); down [E, H, F]; out float32
-    [n, H]; shared [n, H] or float partial sums [P, n, H]."""
+    [n, H]; shared [n, H] or float partial sums [P, n, H].  h [n, H]: the experts' input, which is the output of an
+    identity expert (idx[t, k] >= E; without h such pairs add nothing)."""
     _need(act, "experts act", shape=(None, None, None))
     n, top, F = act.shape
     _need(down, "experts down", act.dtype, (None, None, F))
-    H = down.shape[1]
+    E, H = down.shape[0], down.shape[1]
+    ldh = _ld(h, "experts input") if h is not None else 0
+    if h is not None and (h.dtype != act.dtype or tuple(h.shape) != (n, H)):
+        raise KernelError(f"experts input: {h.dtype} {tuple(h.shape)}, expected {act.dtype} {(n, H)}")
     _need(idx, "chosen experts", torch.int32, (n, top))
     _need(weights, "expert weights", torch.float32, (n, top))
     _need(out, "experts out", torch.float32, (n, H))
@@ -1132,7 +1277,8 @@ def moe_down(act: torch.Tensor, down: torch.Tensor, idx: torch.Tensor, weights: 
         _need(shared_gate, "shared gate", torch.float32, (n,))
     _check(_fn("moe", "cpmcu_moe_down")(_p(act), c_int(_code(act)), _p(down), _p(idx), _p(weights), _p(shared),
                                         c_int(_code(shared) if shared is not None else 0), c_int(sp), c_long(sstr),
-                                        _p(shared_gate), _p(out), c_int(n), c_int(H), c_int(F), c_int(top), _stream()))
+                                        _p(shared_gate), _p(h), c_long(ldh), c_int(E), _p(out), c_int(n), c_int(H),
+                                       c_int(F), c_int(top), _stream()))
 
 
 MOE_TILE = 64
@@ -1154,7 +1300,7 @@ def moe_experts_mfma(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
                      n_tiles: torch.Tensor, shared: Optional[torch.Tensor] = None,
                      shared_gate: Optional[torch.Tensor] = None, activation="silu"):
     """moe_gated + moe_down for steps of many tokens, bf16 on the matrix cores: the (token, expert) pairs are grouped
-    by expert into tiles of MOE_TILE rows.  Scratch: act bf16 [n, top, F], y bf16 [n, top, H], rows int32
+    by expert into tiles of MOE_TILE rows (pairs of identity experts, idx >= E, have none: they add h).  Scratch: act bf16 [n, top, F], y bf16 [n, top, H], rows int32
     [tiles * MOE_TILE], tile_expert int32 [tiles], n_tiles int32 [1], tiles >= moe_tiles(n, top, E)."""
     ldh = _ld(h, "experts input")
     n, H = h.shape
@@ -1183,37 +1329,81 @@ def moe_experts_mfma(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
         *_act(activation), _stream()))
 
 
-def latent_store(proj: torch.Tensor, q_out: torch.Tensor, nh: int, dim: int, rot: int, rank: int,
-                 norm_w: Optional[torch.Tensor], eps: float, positions: torch.Tensor, tok_slot: torch.Tensor,
-                 inv_freq: Optional[torch.Tensor], mag: float, kpool: Optional[torch.Tensor],
-                 vpool: Optional[torch.Tensor], page_table: Optional[torch.Tensor], page_size: int,
-                 write_cache: bool = True):
-    """Latent attention's steps between projection and attention in one launch.  A row of proj is
-    [nh heads of (dim plain | rot rotated) | rank + rot of the down projection (if write_cache) | ...]:
-    every head's rotated part goes, rotated, to q_out[t, head, rank:rank+rot] (q_out [n, nh*(rank+rot)]); with
-    write_cache the latent rmsnorm(down[:rank]) * norm_w goes into the key pages (features 0..rank) and the value
-    pages, and down[rank:], rotated, into the key pages behind it."""
-    ld = _ld(proj, "latent projection")
-    n = proj.shape[0]
-    if proj.shape[1] < nh * (dim + rot) + (rank + rot if write_cache else 0):
-        raise KernelError(f"latent_store: rows of {proj.shape[1]} are too short")
-    _need(q_out, "latent q_out", proj.dtype, (n, nh * (rank + rot)))
-    _need(positions, "latent positions", torch.int32, (n,))
+def latent_store(q_out: Optional[torch.Tensor], nh: int, dim: int, rot: int, rank: int, eps: float, positions: torch.Tensor,
+                 tok_slot: torch.Tensor, inv_freq: Optional[torch.Tensor], mag: float, q_src: Optional[torch.Tensor] = None,
+                 down: Optional[torch.Tensor] = None, norm_w: Optional[torch.Tensor] = None,
+                 kpool: Optional[torch.Tensor] = None, vpool: Optional[torch.Tensor] = None,
+                 page_table: Optional[torch.Tensor] = None, page_size: int = 0, cq_src: Optional[torch.Tensor] = None,
+                 cq_norm_w: Optional[torch.Tensor] = None, cq_out: Optional[torch.Tensor] = None, interleaved: bool = False):
+    """Latent attention's steps between its products and its attention, in one launch; what is not given is left out:
+    * q_src (rows of nh heads of (dim plain | rot rotated)): every head's rotated part goes, rotated, to
+      q_out[t, head, rank:rank+rot] (q_out [n, nh*(rank+rot)]);
+    * down (rows of rank + rot): the latent rmsnorm(down[:rank]) * norm_w goes into the key pages (features 0..rank)
+      and the value pages, and down[rank:], rotated, into the key pages behind it;
+    * cq_src (rows of q_rank): the query latent cq_out [n, q_rank] = rmsnorm(cq_src) * cq_norm_w.
+    The sources may be column slices of wider products.  ``interleaved``: the rotation pairs neighbouring features."""
+    _need(positions, "latent positions", torch.int32, (None,))
+    n = positions.shape[0]
+    given = [t for t in (q_src, down, cq_src) if t is not None]
+    if not given:
+        raise KernelError("latent_store: nothing to do")
+    dt = given[0].dtype
+    if any(t.dtype != dt or t.shape[0] != n for t in given):
+        raise KernelError("latent_store: the sources have one element type and a row a token")
+    ldq = ldd = ldc = 0
     if rot:
         _need(inv_freq, "latent inv_freq", torch.float32, (rot // 2,))
-    tw = pk = pv = 0
-    if write_cache:
+    if q_src is not None:
+        ldq = _ld(q_src, "latent queries")
+        if q_src.shape[1] < nh * (dim + rot):
+            raise KernelError(f"latent_store: query rows of {q_src.shape[1]} are too short")
+        _need(q_out, "latent q_out", dt, (n, nh * (rank + rot)))
+    tw = pk = pv = q_rank = 0
+    if down is not None:
+        ldd = _ld(down, "latent down projection")
+        if down.shape[1] < rank + rot:
+            raise KernelError(f"latent_store: rows of {down.shape[1]} are too short")
         _need(norm_w, "latent norm weight", torch.float32, (rank,))
         _need(tok_slot, "latent token slots", torch.int32, (n,))
         _need(page_table, "latent page table", torch.int32, (None, None))
-        _need(kpool, "latent key pool", proj.dtype, (None, page_size, None))
-        _need(vpool, "latent value pool", proj.dtype, (kpool.shape[0], page_size, None))
+        _need(kpool, "latent key pool", dt, (None, page_size, None))
+        _need(vpool, "latent value pool", dt, (kpool.shape[0], page_size, None))
         tw, pk, pv = page_table.shape[1], kpool.shape[2], vpool.shape[2]
+    if cq_src is not None:
+        ldc, q_rank = _ld(cq_src, "query latent"), cq_src.shape[1]
+        _need(cq_norm_w, "query latent norm weight", torch.float32, (q_rank,))
+        _need(cq_out, "query latent out", dt, (n, q_rank))
+    cache = down is not None
     _check(_fn("attention_general", "cpmcu_latent_store")(
-        _p(proj), c_long(ld), c_int(_code(proj)), _p(q_out), c_int(n), c_int(nh), c_int(dim), c_int(rot), c_int(rank),
-        _p(norm_w if write_cache else None), c_float(eps), _p(positions), _p(tok_slot), _p(inv_freq), c_float(mag),
-        _p(kpool if write_cache else None), _p(vpool if write_cache else None), _p(page_table if write_cache else None),
-        c_int(tw), c_int(page_size), c_int(pk), c_int(pv), c_int(1 if write_cache else 0), _stream()))
+        _p(q_src), c_long(ldq), _p(down), c_long(ldd), _p(cq_src), c_long(ldc), c_int(_DT[dt]), _p(q_out), c_int(n),
+        c_int(nh), c_int(dim), c_int(rot), c_int(rank), _p(norm_w if cache else None), c_float(eps), _p(cq_out),
+        _p(cq_norm_w), c_int(q_rank), _p(positions), _p(tok_slot), _p(inv_freq), c_float(mag),
+        c_int(1 if interleaved else 0), _p(kpool if cache else None), _p(vpool if cache else None),
+        _p(page_table if cache else None), c_int(tw), c_int(page_size), c_int(pk), c_int(pv), _stream()))
+
+
+def head_output(o: torch.Tensor, out: torch.Tensor, nh: int, dv: int, positions: Optional[torch.Tensor] = None,
+                inv_freq: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, interleaved: bool = False):
+    """Between attention and output projection: o [n, nh*dv] (float32, or out's type) -> out [n, nh*dv].  With inv_freq
+    (float32 [dv/2]) every head is turned back by its token's position (the values were cached rotated: pairs
+    (i, i + dv/2), or neighbours when interleaved); with gate [n, nh] (out's type, may be a column slice) head h is
+    multiplied by sigmoid(gate[:, h])."""
+    _need(o, "heads", shape=(None, nh * dv))
+    n = o.shape[0]
+    _need(out, "heads out", shape=(n, nh * dv))
+    if inv_freq is not None:
+        if dv % 2:
+            raise KernelError(f"head_output: rotated values have an even size ({dv})")
+        _need(inv_freq, "value inv_freq", torch.float32, (dv // 2,))
+        _need(positions, "heads positions", torch.int32, (n,))
+    ldg = 0
+    if gate is not None:
+        ldg = _ld(gate, "head gate")
+        if gate.dtype != out.dtype or tuple(gate.shape) != (n, nh):
+            raise KernelError(f"head gate: {gate.dtype} {tuple(gate.shape)}, expected {out.dtype} {(n, nh)}")
+    _check(_fn("attention_general", "cpmcu_head_output")(_p(o), c_int(_code(o)), _p(out), c_int(_code(out)), c_int(n),
+                                                         c_int(nh), c_int(dv), _p(positions), _p(inv_freq),
+                                                         c_int(1 if interleaved else 0), _p(gate), c_long(ldg), _stream()))
 
 
 def _value_heads(nkv: int, v_share: int) -> int:
@@ -1258,7 +1448,8 @@ def attention_general(q: torch.Tensor, out: torch.Tensor, nh: int, nkv: int, hdk
 def gemm_heads(x: torch.Tensor, x_off: int, x_head_stride: int, w: torch.Tensor, out: torch.Tensor, out_off: int,
                out_head_stride: int, gate: Optional[torch.Tensor] = None, plain: bool = False):
     """out[m, out_off + h*out_head_stride + :N] = x[m, x_off + h*x_head_stride + :K] . w[h]^T for every head h;
-    w [H, N, K].  With ``gate`` [m, H] head h's rows are multiplied by sigmoid(gate[m, h]).  bf16 runs on the
+    w [H, N, K].  With ``gate`` [m, H] head h's rows are multiplied by sigmoid(gate[m, h]), with a gate [m, H*N] element
+    by element (heads side by side).  bf16 runs on the
     matrix cores when K and the strides of x are multiples of 8 (``plain``: the scalar kernel all the same)."""
     ldx, ldy = _ld(x, "heads x"), _ld(out, "heads out")
     M = x.shape[0]
@@ -1268,22 +1459,23 @@ def gemm_heads(x: torch.Tensor, x_off: int, x_head_stride: int, w: torch.Tensor,
         raise KernelError(f"gemm_heads: {H} heads of {K} features from column {x_off} do not fit rows of {x.shape[1]}")
     if out.shape[0] != M or out_off < 0 or out_off + (H - 1) * out_head_stride + N > out.shape[1]:
         raise KernelError(f"gemm_heads: {H} heads of {N} features to column {out_off} do not fit {tuple(out.shape)}")
-    ldg = 0
+    ldg, wide = 0, False
     if gate is not None:
         ldg = _ld(gate, "heads gate")
-        if gate.dtype != x.dtype or tuple(gate.shape) != (M, H):
-            raise KernelError(f"heads gate: {gate.dtype} {tuple(gate.shape)}, expected {x.dtype} {(M, H)}")
+        wide = gate.shape[1] != H
+        if gate.dtype != x.dtype or tuple(gate.shape) not in ((M, H), (M, H * N)):
+            raise KernelError(f"heads gate: {gate.dtype} {tuple(gate.shape)}, expected {x.dtype} {(M, H)} or {(M, H * N)}")
     xp = c_void_p(x.data_ptr() + x_off * x.element_size())
     op = c_void_p(out.data_ptr() + out_off * out.element_size())
     if (x.dtype == torch.bfloat16 and out.dtype == torch.bfloat16 and not plain and K % 8 == 0 and ldx % 8 == 0
             and x_head_stride % 8 == 0 and xp.value % 16 == 0 and w.data_ptr() % 16 == 0):
         _check(_fn("gemm", "cpmcu_gemm_nt_heads_mfma")(xp, c_long(ldx), c_long(x_head_stride), _p(w), op, c_long(ldy),
-                                                       c_long(out_head_stride), _p(gate), c_long(ldg), c_int(M),
-                                                       c_int(H), c_int(N), c_int(K), _stream()))
+                                                       c_long(out_head_stride), _p(gate), c_long(ldg),
+                                                       c_int(1 if wide else 0), c_int(M), c_int(H), c_int(N), c_int(K), _stream()))
         return
     _check(_fn("gemm", "cpmcu_gemm_nt_heads")(xp, c_long(ldx), c_long(x_head_stride), _p(w), op, c_long(ldy),
-                                              c_long(out_head_stride), _p(gate), c_long(ldg), c_int(_code(x)),
-                                              c_int(_code(out)), c_int(M), c_int(H), c_int(N), c_int(K), _stream()))
+                                              c_long(out_head_stride), _p(gate), c_long(ldg),
+                                              c_int(1 if wide else 0), c_int(_code(x)), c_int(_code(out)), c_int(M), c_int(H), c_int(N), c_int(K), _stream()))
 
 
 def argmax(logits: torch.Tensor, out: torch.Tensor):
@@ -1697,7 +1889,7 @@ def attention_any(q, out, nh, nkv, hdk, hdv, scale, kpool, vpool, page_table, pa
     the caller applies it itself after the other kernels.  softcap c > 0: scaled scores pass c tanh(s / c)."""
     pool_hdv = vpool.shape[2] // _value_heads(nkv, v_share)
     if (hdk == hdv and chunk == 0 and window == 0 and sink is None and hdk <= 256 and hdk % 16 == 0
-            and kpool.shape[2] == nkv * hdk and v_share == 1 and not softcap):
+            and kpool.shape[2] == nkv * hdk and v_share == 1 and not softcap and out.dtype == q.dtype):
         attention(q, out, nh, nkv, hdk, scale, kpool, vpool, page_table, page_size, ctx)
         return False
     if attention_general_mfma_ok(q, hdk, hdv, page_size):

@@ -13,5 +13,9 @@ from .delta import GatedDeltaMixer
 from .parallel import ParallelMixer
 from .linear_attention import DecayLinearAttention
 from .ffn import GatedFFN, PolyNormFFN, RoutedExpertsFFN
-from .block import HyperConnectionBlock, ParallelGatedBlock, ParallelScaledBlock, PreNormBlock, SandwichNormBlock
+from .input_conv import InputConvolution
+from .token_input import TokenInput, TokenTable
+from .loop_input import LoopInput
+from .block import (HyperConnectionBlock, ParallelBlock, ParallelGatedBlock, ParallelScaledBlock, PreNormBlock,
+                    SandwichNormBlock)
 from .embedding import LMHead, TokenEmbedding

@@ -241,7 +241,9 @@ class GeneralAttention(Mixer):
       'sink'               one number a head: exp(sink) joins the softmax's denominator as a term that has no key,
                            no value and no scale;
       'gate'               an output gate: the heads side by side are multiplied element by element with
-                           sigmoid(W_gate h) before the output projection (its rows ride in the q/k/v product).
+                           sigmoid(W_gate h) before the output projection (its rows ride in the q/k/v product);
+      'head_gate'          an output gate of one number a head, sigmoid(W_gate h)_head, instead;
+      'temp'               one number a head that multiplies its (scaled) scores.
       'q_conv', 'k_conv', 'v_conv'   with ``conv_taps`` > 0: a short causal convolution over time on every channel of
                            q, k and v ([channels, taps], the last tap the current token's, zeros before the start,
                            no bias, no activation) directly behind the projection; the last taps - 1 projected rows
@@ -250,6 +252,8 @@ class GeneralAttention(Mixer):
     root, no weight) after the rotation.
     The rotation pairs the features that ``position.pairs`` says ('halves': i with i + r/2 of the r rotated features;
     'interleaved': 2i with 2i + 1).
+    ``value_position``: a rotation of all value features (no magnitude, the pairs of ``position``): the value of key j is
+    cached rotated by j, and a head's output at position p is turned back by p, before any gate.
     ``score_softcap`` c: a scaled score s enters the softmax as c tanh(s / c).
     Without 'v' the values are the keys as projected (with their bias, before norm and rotation): value_dim
     must equal key_dim."""
@@ -257,7 +261,8 @@ class GeneralAttention(Mixer):
     def __init__(self, names: Mapping[str, str], hidden_size: int, num_heads: int, num_kv_heads: int, key_dim: int,
                  value_dim: int, position: Optional[PositionEncoding], scale: float, mask_chunk: Optional[int] = None,
                  mask_window: Optional[int] = None, mask_keep_first: int = 0, norm_eps: float = 0.0,
-                 unit_norm_after_rotation: bool = False, score_softcap: Optional[float] = None, conv_taps: int = 0):
+                 unit_norm_after_rotation: bool = False, score_softcap: Optional[float] = None, conv_taps: int = 0,
+                 value_position: Optional[PositionEncoding] = None):
         if num_heads % num_kv_heads:
             raise ValueError(f"attention: {num_heads} heads are not a multiple of {num_kv_heads} kv heads")
         if unit_norm_after_rotation and (names.get("q_norm") or names.get("k_norm")):
@@ -281,8 +286,15 @@ class GeneralAttention(Mixer):
         self.taps = int(conv_taps)
         self.names = dict(names)
         self.values_are_keys = "v" not in self.names
-        if self.taps and (self.values_are_keys or self.names.get("gate")):
+        if self.taps and (self.values_are_keys or self.names.get("gate") or self.names.get("head_gate")):
             raise ValueError("attention: the convolution goes with q, k and v of their own and no output gate")
+        if self.names.get("gate") and (self.names.get("head_gate") or value_position is not None):
+            raise ValueError("attention: an output gate a feature goes with no gate a head and no rotated values")
+        if value_position is not None:
+            if self.values_are_keys or value_dim % 2 or (position is not None and value_position.pairs != position.pairs):
+                raise ValueError("attention: rotated values have an even size, heads of their own and the keys' layout of pairs")
+            self.interleaved = value_position.pairs == "interleaved"
+        self.value_position = value_position
         if self.values_are_keys and value_dim != key_dim:
             raise ValueError(f"attention: values that are the keys have the keys' size ({value_dim}, {key_dim})")
         self.hidden_size, self.nh, self.nkv, self.dk, self.dv = hidden_size, num_heads, num_kv_heads, key_dim, value_dim
@@ -299,22 +311,29 @@ class GeneralAttention(Mixer):
             self.gate_off = sum(r for _, r in stacked)
             stacked.append((self.names["gate"], num_heads * value_dim))
             biases.append(None)
+        self.head_gate_off = None
+        if self.names.get("head_gate"):
+            self.head_gate_off = sum(r for _, r in stacked)
+            stacked.append((self.names["head_gate"], num_heads))
+            biases.append(None)
         self.qkv = Linear(stacked, hidden_size, bias_names=biases if any(biases) else None)
         self.o = Linear([(self.names["out"], hidden_size)], num_heads * value_dim,
                         bias_names=[self.names["out_bias"]] if self.names.get("out_bias") else None)
         # what the plain rotate-and-store kernel does not do
         self._extras = bool(any(biases) or self.names.get("q_norm") or self.names.get("k_norm") or self.values_are_keys
-                            or self.norm_after or self.taps)
+                            or self.norm_after or self.taps or self.names.get("temp") or value_position is not None)
         self.conv_widths = (num_heads * key_dim, num_kv_heads * key_dim, num_kv_heads * value_dim)
 
     def parts(self) -> List[Part]:
-        return [self.qkv, self.o] + ([self.position] if self.position is not None else [])
+        return [self.qkv, self.o] + [p for p in (self.position, self.value_position) if p is not None]
 
     def weight_specs(self):
         from .base import WeightSpec
         specs = [WeightSpec(self.names[k], (self.dk,), "norm") for k in ("q_norm", "k_norm") if self.names.get(k)]
         if self.names.get("sink"):
             specs.append(WeightSpec(self.names["sink"], (self.nh,), "small"))
+        if self.names.get("temp"):
+            specs.append(WeightSpec(self.names["temp"], (self.nh,), "norm"))
         if self.taps:
             specs += [WeightSpec(self.names[k], (w, self.taps), "conv_taps")
                       for k, w in zip(("q_conv", "k_conv", "v_conv"), self.conv_widths)]
@@ -323,7 +342,7 @@ class GeneralAttention(Mixer):
     def bind(self, tensors: Mapping[str, torch.Tensor], rt: Runtime):
         self.rt = rt
         f = lambda k: tensors[self.names[k]].to(torch.float32).contiguous() if self.names.get(k) else None
-        self.q_norm, self.k_norm, self.sink = f("q_norm"), f("k_norm"), f("sink")
+        self.q_norm, self.k_norm, self.sink, self.temp = f("q_norm"), f("k_norm"), f("sink"), f("temp")
         if self.taps:
             self.conv_w = torch.cat([f("q_conv"), f("k_conv"), f("v_conv")], 0).contiguous()
 
@@ -354,8 +373,14 @@ class GeneralAttention(Mixer):
             raise ValueError(f"attention: the rotation covers {rd} features, a head has {dk}")
         if self.taps and not writes_cache:
             raise ValueError("attention: a run that reads another run's cache has no convolution state of its own")
+        gated = self.gate_off is not None or self.head_gate_off is not None
+        v_freq = None
+        if self.value_position is not None:
+            v_freq = self.value_position.rotary_params()[0]
+            if 2 * v_freq.shape[0] != dv:
+                raise ValueError(f"attention: the values' rotation covers {2 * v_freq.shape[0]} features, a value has {dv}")
         with ctx.timed("attn_qkv_rope"):
-            qkv = self.qkv.forward(h, ctx, "attn.qkv", rows=None if (writes_cache or self.gate_off is not None) else nh * dk)
+            qkv = self.qkv.forward(h, ctx, "attn.qkv", rows=None if (writes_cache or gated) else nh * dk)
             if self.taps:
                 # the projected rows mixed over time, in float; the slot's state moves on to the step's last rows
                 mixed = ctx.ws.get("attn.conv", (n, sum(self.conv_widths)), torch.float32)
@@ -368,12 +393,15 @@ class GeneralAttention(Mixer):
                                           cache.streams["k"], cache.streams["v"], cache.page_table, cache.page_size,
                                           write_kv=writes_cache, bias=self.qkv.bias, q_norm=self.q_norm,
                                           k_norm=self.k_norm, eps=self.norm_eps, values_from_keys=self.values_are_keys,
-                                          norm_after=self.norm_after, interleaved=self.interleaved)
+                                          norm_after=self.norm_after, interleaved=self.interleaved, q_scale=self.temp,
+                                          v_inv_freq=v_freq)
             else:
                 ops.qkv_rotate_store(qkv, q, nh, nkv, dk, dv, rd, ctx.positions, ctx.tok_slot, inv_freq, mag,
                                      cache.streams["k"], cache.streams["v"], cache.page_table, cache.page_size,
                                      write_kv=writes_cache, interleaved=self.interleaved)
-        out = ctx.ws.get("attn.out", (n, nh * dv), self.rt.dtype)
+        # heads that pass head_output leave the attention as float
+        finish = v_freq is not None or self.head_gate_off is not None
+        out = ctx.ws.get("attn.heads" if finish else "attn.out", (n, nh * dv), torch.float32 if finish else self.rt.dtype)
         gate = qkv[:, self.gate_off:self.gate_off + nh * dv] if self.gate_off is not None else None
         with ctx.timed("attn_core"):
             # the matrix-core kernel (and the merge of split keys) applies the gate as it writes
@@ -385,6 +413,11 @@ class GeneralAttention(Mixer):
                 gated = ctx.ws.get("attn.gated", (n, nh * dv), self.rt.dtype)
                 ops.sigmoid_gate(out, gate, gated)
                 out = gated
+        if finish:
+            with ctx.timed("attn_gate"):
+                heads, out = out, ctx.ws.get("attn.out", (n, nh * dv), self.rt.dtype)
+                head_gate = qkv[:, self.head_gate_off:self.head_gate_off + nh] if self.head_gate_off is not None else None
+                ops.head_output(heads, out, nh, dv, ctx.positions, v_freq, head_gate, interleaved=self.interleaved)
         with ctx.timed("attn_o"):
             branch = self.o.forward(out, ctx, "attn.o", out_dtype=torch.float32, partials=True)
         return BiasedBranch(branch, self.o.bias, ctx, "attn.o") if self.o.bias is not None else branch

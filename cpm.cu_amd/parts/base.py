@@ -190,6 +190,21 @@ class BiasedBranch:
         return self._value
 
 
+class ReplacingBranch:
+    """What takes the residual's place: x <- ``branch`` + ``bias`` (tensor [n, H] or float partial sums [P, n, H];
+    bias float32 [H] or None), left pending like every branch for the norm that follows (Norm.takes_replacing_branch);
+    for everybody else ``evaluate()`` does it and leaves nothing to add (None)."""
+
+    def __init__(self, x: torch.Tensor, branch: torch.Tensor, bias: Optional[torch.Tensor] = None):
+        self.x, self.branch, self.bias = x, branch, bias
+
+    def evaluate(self) -> None:
+        from .. import ops
+        if self.branch is not None:
+            ops.norm_rows(self.x, None, None, branch=self.branch, branch_bias=self.bias, replace=True)
+            self.branch = None
+
+
 class StreamsBranch:
     """A sub-layer's result that joins a residual of several streams (hyper-connections): all streams at once,
     x_t <- sum_s ``mix``[s, t] x_s + ``out``[t] * ``branch`` (mix float32 [S, S] indexed [from, to], out float32
@@ -208,7 +223,9 @@ class StreamsBranch:
 
 def branch_tensor(branch):
     """The branch as a tensor (or None), whatever form it was handed over in."""
-    return branch.evaluate() if isinstance(branch, (DeferredBranch, NormedBranch, BiasedBranch)) else branch
+    if isinstance(branch, (DeferredBranch, NormedBranch, BiasedBranch, ReplacingBranch)):
+        return branch.evaluate()
+    return branch
 
 
 def branch_for(norm: "Norm", branch):
@@ -219,6 +236,8 @@ def branch_for(norm: "Norm", branch):
     if isinstance(branch, NormedBranch) and not norm.takes_normed_branch:
         return branch.evaluate()
     if isinstance(branch, BiasedBranch) and not norm.takes_biased_branch:
+        return branch.evaluate()
+    if isinstance(branch, ReplacingBranch) and not norm.takes_replacing_branch:
         return branch.evaluate()
     return branch
 
@@ -309,6 +328,18 @@ class Norm(Part):
     takes_normed_branch = False
     # True if forward and forward_unscaled accept a BiasedBranch as ``branch``
     takes_biased_branch = False
+    # True if forward and forward_unscaled accept a ReplacingBranch as ``branch``
+    takes_replacing_branch = False
+
+    # True if forward accepts ``out_dtype=`` (the element type of the normed rows; None: the engine's)
+    takes_out_dtype = False
+
+    def forward_convolved(self, x: torch.Tensor, branch, branch_scale: float, ctx: StepContext, convs, conv_state,
+                          tags: Sequence[str]) -> Optional[List[torch.Tensor]]:
+        """For a step in which every row is a sequence's only token, and a norm that knows a kernel for it: add the
+        branch as forward does, norm, and run the short convolutions ``convs`` over the normed rows, h + conv(h) each,
+        with the sequences' earlier rows from ``conv_state`` (ops.norm_rows).  None: the caller does it in steps."""
+        return None
 
     def forward_streams(self, x: torch.Tensor, pending: Optional["StreamsBranch"], read: Optional[torch.Tensor],
                         ctx: StepContext, rows: Optional[torch.Tensor] = None, tag: str = "norm") -> torch.Tensor:
@@ -391,6 +422,10 @@ def forward_declares(part: Part, flag: str) -> bool:
 
 class Block(Part):
     mixer: Mixer
+
+    def cache_needs(self) -> CacheNeeds:
+        """What a run of this block keeps per sequence: its mixer's needs, and the block's own."""
+        return self.mixer.cache_needs()
 
     def forward(self, stream: ResidualStream, ctx: StepContext, cache: Optional[CacheView], writes_cache: bool = True):
         raise NotImplementedError

@@ -8,16 +8,26 @@ model's final norm).
 """
 from __future__ import annotations
 
+from dataclasses import replace
 from typing import List, Optional
 
-from ..cache.paged import CacheView
+from ..cache.paged import CacheNeeds, CacheView
 import torch
 
 from .. import ops
 from .base import (BLOCKS, BiasedBranch, Block, DeferredBranch, FeedForward, Mixer, Norm, NormedBranch, Part,
                    ResidualStream, Runtime, StepContext, StreamsBranch, WeightSpec, branch_for, branch_tensor,
                    forward_declares)
+from .input_conv import InputConvolution
 from .linear import Linear
+from .token_input import TokenInput
+
+
+def _with_bias(branch):
+    """A sub-layer's result as (tensor, bias or None)."""
+    if isinstance(branch, BiasedBranch):
+        return branch.branch, branch.bias
+    return branch_tensor(branch), None
 
 
 @BLOCKS.register("pre_norm")
@@ -141,22 +151,16 @@ class ParallelGatedBlock(Block):
     def parts(self) -> List[Part]:
         return [self.norm, self.mixer] + ([self.feed_forward] if self.feed_forward is not None else []) + [self.gates]
 
-    @staticmethod
-    def _with_bias(branch):
-        if isinstance(branch, BiasedBranch):
-            return branch.branch, branch.bias
-        return branch_tensor(branch), None
-
     def forward(self, stream: ResidualStream, ctx: StepContext, cache: Optional[CacheView], writes_cache: bool = True):
         with ctx.timed("norm"):
             h = self.norm.forward(stream.x, branch_for(self.norm, stream.take_pending()), stream.pending_scale, ctx,
                                   tag="block.h")
         with ctx.timed("attn"):
-            a, a_bias = self._with_bias(self.mixer.forward(h, ctx, cache, writes_cache))
+            a, a_bias = _with_bias(self.mixer.forward(h, ctx, cache, writes_cache))
         f = f_bias = None
         if self.feed_forward is not None:
             with ctx.timed("ffn"):
-                f, f_bias = self._with_bias(self.feed_forward.forward(h, ctx))
+                f, f_bias = _with_bias(self.feed_forward.forward(h, ctx))
         with ctx.timed("gates"):
             few = h.shape[0] <= ops.SKINNY_MAX_ROWS
             g = self.gates.forward(h, ctx, "block.gates", out_dtype=torch.float32 if few else None)
@@ -192,27 +196,78 @@ class ParallelScaledBlock(Block):
     def bind(self, tensors, rt: Runtime):
         self.scales = [tensors[name].to(torch.float32).contiguous() for name in self.scale_names]
 
-    @staticmethod
-    def _with_bias(branch):
-        if isinstance(branch, BiasedBranch):
-            return branch.branch, branch.bias
-        return branch_tensor(branch), None
-
     def forward(self, stream: ResidualStream, ctx: StepContext, cache: Optional[CacheView], writes_cache: bool = True):
         with ctx.timed("norm"):
             h = self.norm.forward(stream.x, branch_for(self.norm, stream.take_pending()), stream.pending_scale, ctx,
                                   tag="block.h")
         with ctx.timed("attn"):
-            a, a_bias = self._with_bias(self.mixer.forward(h, ctx, cache, writes_cache))
+            a, a_bias = _with_bias(self.mixer.forward(h, ctx, cache, writes_cache))
         f = f_bias = None
         if self.feed_forward is not None:
             with ctx.timed("ffn"):
-                f, f_bias = self._with_bias(self.feed_forward.forward(h, ctx))
+                f, f_bias = _with_bias(self.feed_forward.forward(h, ctx))
         with ctx.timed("layer_scale"):
             out = ctx.ws.get("block.scaled", (h.shape[0], self.hidden_size), torch.float32)
             ops.scaled_branches(a, a_bias, self.scales[0], 1.0, f, f_bias, self.scales[1] if f is not None else None, 1.0,
                                 out)
         stream.pending = out
+        stream.pending_scale = 1.0
+
+
+@BLOCKS.register("parallel")
+class ParallelBlock(Block):
+    """One norm a layer, both sub-layers read its output and their results join the residual as they are:
+
+        h = norm(x);  x += Mixer(h + conv1(h)) + FeedForward(h + conv2(h))
+
+    ``input_conv``: the short convolutions on what the sub-layers read (absent: both read h itself); what they remember
+    is fixed-size state of the run's cache entry.  ``token_input``: what the layer adds for the tokens themselves
+    afterwards, x += norm of its result.  A layer may have no feed-forward.  The last result is left pending for the
+    norm that follows."""
+
+    def __init__(self, norm: Norm, mixer: Mixer, feed_forward: Optional[FeedForward], hidden_size: int,
+                 input_conv: Optional[InputConvolution] = None, token_input: Optional[TokenInput] = None):
+        if input_conv is not None and len(input_conv.names) != (2 if feed_forward is not None else 1):
+            raise ValueError("parallel: one input convolution for every sub-layer")
+        self.norm, self.mixer, self.feed_forward, self.hidden_size = norm, mixer, feed_forward, hidden_size
+        self.input_conv, self.token_input = input_conv, token_input
+
+    def parts(self) -> List[Part]:
+        return [p for p in (self.norm, self.input_conv, self.mixer, self.feed_forward, self.token_input) if p is not None]
+
+    def cache_needs(self) -> CacheNeeds:
+        needs = self.mixer.cache_needs()
+        if self.input_conv is not None:
+            needs = replace(needs, state=needs.state + self.input_conv.state())
+        return needs
+
+    def bind(self, tensors, rt: Runtime):
+        self.rt = rt
+
+    def forward(self, stream: ResidualStream, ctx: StepContext, cache: Optional[CacheView], writes_cache: bool = True):
+        if self.input_conv is not None and not writes_cache:
+            raise ValueError("parallel: a run that reads another run's cache has no convolution state of its own")
+        with ctx.timed("norm"):
+            if self.input_conv is not None:
+                hs = self.input_conv.forward(self.norm, stream, ctx, cache)
+            else:
+                hs = [self.norm.forward(stream.x, branch_for(self.norm, stream.take_pending()), stream.pending_scale, ctx,
+                                        tag="block.h")]
+        with ctx.timed("attn"):
+            a, a_bias = _with_bias(self.mixer.forward(hs[0], ctx, cache, writes_cache))
+        f = f_bias = None
+        if self.feed_forward is not None:
+            with ctx.timed("ffn"):
+                f, f_bias = _with_bias(self.feed_forward.forward(hs[-1], ctx))
+        x = stream.x
+        with ctx.timed("residual"):
+            if self.token_input is None:
+                out = ctx.ws.get("block.sum", tuple(x.shape), torch.float32)
+                ops.scaled_branches(a, a_bias, None, 1.0, f, f_bias, None, 1.0, out)
+            else:
+                out = ctx.ws.get("block.x", tuple(x.shape), self.rt.dtype)
+                ops.add_rows(x, a, a_bias, f, f_bias, out)
+        stream.pending = out if self.token_input is None else self.token_input.forward(out, ctx)
         stream.pending_scale = 1.0
 
 

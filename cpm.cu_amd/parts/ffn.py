@@ -98,22 +98,27 @@ class RoutedExpertsFFN(FeedForward):
     ``keep`` best groups can be chosen.  The chosen experts' outputs are added with weights s / (sum of the chosen s +
     1e-20) * ``weight_scale``.  A shared expert (``shared_size``) runs for every token and is added, times
     sigmoid(w . h), one number a token, if ``names`` holds 'shared_scale'.  ``activation`` / ``shared_activation``:
-    the experts' and the shared expert's nonlinearity as GatedFFN takes it.
+    the experts' and the shared expert's nonlinearity as GatedFFN takes it.  Without ``normalize`` the weights are
+    s * ``weight_scale``.  ``identity``: so many further rows of the router (and of the correction) are identity
+    experts, which have no tensors and give the layer's input back.
 
     ``names``: 'router', 'correction' (or absent), 'expert' (a format with {e} for the expert's number and {part}
     for gate / up / down), and for the shared expert 'shared_gate', 'shared_up', 'shared_down', 'shared_scale'."""
 
     def __init__(self, names: Mapping[str, str], hidden_size: int, expert_size: int, experts: int, top: int,
                  groups: Optional[Tuple[int, int]] = None, shared_size: Optional[int] = None, score: str = "softmax",
-                 group_score: str = "max", weight_scale: float = 1.0, activation="silu", shared_activation=None):
-        if experts > ops.MOE_MAX_EXPERTS:
-            raise ValueError(f"routed_experts: {experts} experts (up to {ops.MOE_MAX_EXPERTS} are taken)")
-        if not 0 < top <= experts:
-            raise ValueError(f"routed_experts: {top} of {experts} experts a token")
+                 group_score: str = "max", weight_scale: float = 1.0, activation="silu", shared_activation=None,
+                 normalize: bool = True, identity: int = 0):
+        routes = experts + identity
+        if experts < 1 or identity < 0 or routes > ops.MOE_MAX_EXPERTS:
+            raise ValueError(f"routed_experts: {experts} experts and {identity} identity experts (one to "
+                             f"{ops.MOE_MAX_EXPERTS} in all are taken)")
+        if not 0 < top <= routes:
+            raise ValueError(f"routed_experts: {top} of {routes} experts a token")
         if groups is not None:
             count, keep = groups
-            if count <= 0 or experts % count or not 0 < keep <= count or top > keep * (experts // count):
-                raise ValueError(f"routed_experts: {experts} experts in {count} groups, {keep} kept, {top} chosen")
+            if count <= 0 or routes % count or not 0 < keep <= count or top > keep * (routes // count):
+                raise ValueError(f"routed_experts: {routes} experts in {count} groups, {keep} kept, {top} chosen")
         if score not in ops.MOE_SCORES or group_score not in ops.MOE_GROUP_SCORES:
             raise ValueError(f"routed_experts: score '{score}' ({sorted(ops.MOE_SCORES)}) or group score "
                              f"'{group_score}' ({sorted(ops.MOE_GROUP_SCORES)})")
@@ -122,6 +127,7 @@ class RoutedExpertsFFN(FeedForward):
         except ops.KernelError as e:
             raise ValueError(f"routed_experts: {e}") from None
         self.score, self.group_score, self.weight_scale = score, group_score, float(weight_scale)
+        self.normalize, self.routes = bool(normalize), routes
         self.names = dict(names)
         self.hidden_size, self.expert_size, self.experts, self.top = hidden_size, expert_size, experts, top
         self.groups = tuple(groups) if groups is not None else (1, 1)
@@ -141,9 +147,9 @@ class RoutedExpertsFFN(FeedForward):
 
     def weight_specs(self) -> List[WeightSpec]:
         H, F = self.hidden_size, self.expert_size
-        specs = [WeightSpec(self.names["router"], (self.experts, H))]
+        specs = [WeightSpec(self.names["router"], (self.routes, H))]
         if self.names.get("correction"):
-            specs.append(WeightSpec(self.names["correction"], (self.experts,), "slight"))
+            specs.append(WeightSpec(self.names["correction"], (self.routes,), "slight"))
         for e in range(self.experts):
             specs += [WeightSpec(self._expert(e, "gate"), (F, H)), WeightSpec(self._expert(e, "up"), (F, H)),
                       WeightSpec(self._expert(e, "down"), (H, F))]
@@ -167,11 +173,11 @@ class RoutedExpertsFFN(FeedForward):
         idx = ctx.ws.get("moe.idx", (n, self.top), torch.int32)
         wts = ctx.ws.get("moe.weights", (n, self.top), torch.float32)
         sg = ctx.ws.get("moe.shared_gate", (n,), torch.float32) if self.shared_gated else None
-        logits = ctx.ws.get("moe.logits", (n, self.experts + 1), torch.float32)
+        logits = ctx.ws.get("moe.logits", (n, self.routes + 1), torch.float32)
         with ctx.timed("moe_route"):
             ops.moe_route(h, self.router, self.correction, self.shared_scale, self.groups[0], self.groups[1], self.top,
                           idx, wts, sg, logits, score=self.score, group_score=self.group_score,
-                          weight_scale=self.weight_scale)
+                          weight_scale=self.weight_scale, normalize=self.normalize)
         shared = self.shared.forward(h, ctx) if self.shared is not None else None
         act = ctx.ws.get("moe.act", (n, self.top, self.expert_size), self.rt.dtype)
         out = ctx.ws.get("moe.out", (n, self.hidden_size), torch.float32)
@@ -191,5 +197,5 @@ class RoutedExpertsFFN(FeedForward):
             else:
                 # few tokens: an expert's weights stream once for every token that chose it
                 ops.moe_gated(h, self.gate_up, idx, act, activation=self.activation)
-                ops.moe_down(act, self.down, idx, wts, out, shared, sg)
+                ops.moe_down(act, self.down, idx, wts, out, shared, sg, h=h)
         return out

@@ -81,6 +81,15 @@ class Linear(Part):
         ops.linear(x, w, out, alpha, w_tiled=wt)
         return out
 
+    def forward_float(self, x: torch.Tensor, ctx: StepContext, tag: str) -> torch.Tensor:
+        """x [n, in] -> float32 [n, out], or float partial sums [S, n, out], whatever the number of rows: for a result
+        that takes the place of the residual, which is never rounded to 16 bits."""
+        if x.shape[0] <= ops.SKINNY_MAX_ROWS or x.dtype == torch.float32:
+            return self.forward(x, ctx, tag, out_dtype=torch.float32, partials=True)
+        out = ctx.ws.get(tag, (x.shape[0], self.out_features), torch.float32)
+        torch.mm(x, self.weight.t(), out_dtype=torch.float32, out=out)      # the library's product, summed and left in float
+        return out
+
     def defers(self, x: torch.Tensor) -> bool:
         """Whether, for these rows, a norm could run this product itself (ops.proj_add_norm): only then is it
         worth handing the product over instead of running it."""

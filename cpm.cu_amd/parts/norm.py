@@ -11,8 +11,8 @@ from typing import List, Mapping, Optional
 import torch
 
 from .. import ops
-from .base import (NORMS, BiasedBranch, DeferredBranch, Norm, NormedBranch, Runtime, StepContext, StreamsBranch, WeightSpec,
-                   branch_tensor)
+from .base import (NORMS, BiasedBranch, DeferredBranch, Norm, NormedBranch, ReplacingBranch, Runtime, StepContext,
+                   StreamsBranch, WeightSpec, branch_tensor)
 
 
 @NORMS.register("rms_norm")
@@ -97,6 +97,18 @@ def _streams_norm(norm, x, pending: Optional[StreamsBranch], read, ctx: StepCont
     return out
 
 
+def row_branch(branch, branch_scale: float) -> dict:
+    """A pending branch, in whatever form it was left, as ops.norm_rows takes it."""
+    if isinstance(branch, ReplacingBranch):
+        return {} if branch.branch is None else dict(branch=branch.branch, branch_bias=branch.bias, replace=True)
+    if isinstance(branch, NormedBranch) and isinstance(branch.norm, RMSNorm) and branch_scale == 1.0:
+        return dict(branch=branch_tensor(branch.branch), branch_norm=branch.norm.weight, branch_eps=branch.norm.eps)
+    if isinstance(branch, BiasedBranch) and branch_scale == 1.0:
+        return dict(branch=branch.branch, branch_bias=branch.bias)
+    branch = branch_tensor(branch)
+    return {} if branch is None else dict(branch=branch, branch_scale=branch_scale)
+
+
 @NORMS.register("layer_norm")
 class LayerNorm(Norm):
     """Layer norm with a weight and no bias: y = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w, statistics in
@@ -115,10 +127,16 @@ class LayerNorm(Norm):
         self.rt = rt
 
     takes_biased_branch = True
+    takes_normed_branch = True
+    takes_replacing_branch = True
+    takes_out_dtype = True
 
-    def forward(self, x, branch, branch_scale, ctx: StepContext, rows=None, tag="norm"):
+    def forward(self, x, branch, branch_scale, ctx: StepContext, rows=None, tag="norm", out_dtype=None):
         n_out = x.shape[0] if rows is None else rows.shape[0]
-        out = ctx.ws.get(tag, (n_out, self.hidden_size), self.rt.dtype)
+        out = ctx.ws.get(tag, (n_out, self.hidden_size), out_dtype or self.rt.dtype)
+        if isinstance(branch, (NormedBranch, ReplacingBranch)):
+            ops.norm_rows(x, out, "layer", self.weight, self.eps, rows=rows, **row_branch(branch, branch_scale))
+            return out
         bias = None
         if isinstance(branch, BiasedBranch):
             branch, bias = branch.branch, branch.bias
@@ -129,3 +147,9 @@ class LayerNorm(Norm):
 
     def forward_streams(self, x, pending, read, ctx: StepContext, rows=None, tag="norm"):
         return _streams_norm(self, x, pending, read, ctx, rows, tag, rms=False)
+
+    def forward_convolved(self, x, branch, branch_scale, ctx: StepContext, convs, conv_state, tags):
+        outs = [ctx.ws.get(tag, (x.shape[0], self.hidden_size), self.rt.dtype) for tag in tags]
+        ops.norm_rows(x, outs[0], "layer", self.weight, self.eps, convs=convs, conv_state=conv_state, slots=ctx.tok_slot,
+                      out2=outs[1] if len(outs) > 1 else None, **row_branch(branch, branch_scale))
+        return outs

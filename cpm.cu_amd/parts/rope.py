@@ -1,7 +1,7 @@
 """Rotary position encoding, plain and LongRoPE.
 
 Rotate-half rotation by theta = position * inv_freq[c] (src/model/rotary.cuh:7-34); with ``pairs='interleaved'`` the
-plain encoding pairs neighbouring features (2c, 2c + 1) instead of (c, c + head_dim/2), with the same angles.
+plain and YaRN encodings pair neighbouring features (2c, 2c + 1) instead of (c, c + head_dim/2), with the same angles.
 The reference loads inv_freq once, computed for the engine's whole token budget
 (cpmcu/llm.py:181-191): the choice between LongRoPE's short and long factors is
 static per engine, long iff the engine holds sequences longer than
@@ -75,8 +75,9 @@ class YarnRotaryEncoding(RotaryEncoding):
         freq_i = f_i / factor * ramp_i + f_i * (1 - ramp_i)
     and cos and sin carry the magnitude 0.1 ln(factor) + 1."""
 
-    def __init__(self, head_dim: int, theta: float, factor: float, original: int, fast: float, slow: float):
-        super().__init__(head_dim, theta)
+    def __init__(self, head_dim: int, theta: float, factor: float, original: int, fast: float, slow: float,
+                 pairs: str = "halves"):
+        super().__init__(head_dim, theta, pairs)
         self.factor, self.original, self.fast, self.slow = float(factor), float(original), float(fast), float(slow)
         self.magnitude = 0.1 * math.log(self.factor) + 1.0
 
