@@ -149,13 +149,18 @@ def expert(h, W, p):
 
 def route(h, W, p, r, margins=None):
     """(chosen experts [T, top], weights [T, top]).  ``margins`` (a list) receives, per token, how clear the choice
-    was: the gap between the last choice score taken and the first one left."""
+    was: the gap between the last choice score taken and the first one left, against the two scores' sum (rounding of
+    the router's input moves a softmax score in proportion to itself)."""
     top = int(r["top"])
     s = torch.softmax(h @ W[p + "router"].T, -1)
     c = s + W[p + "correction"]
     ranked, order = c.sort(-1, descending=True)
     if margins is not None:
-        margins.append(ranked[:, top - 1] - ranked[:, top] if top < c.shape[1] else torch.full((h.shape[0],), math.inf, dtype=F64))
+        if top < c.shape[1]:
+            near = s.gather(1, order[:, top - 1:top + 1]).sum(-1)
+            margins.append((ranked[:, top - 1] - ranked[:, top]) / near)
+        else:
+            margins.append(torch.full((h.shape[0],), math.inf, dtype=F64))
     idx = order[:, :top]
     return idx, s.gather(1, idx)
 
@@ -197,9 +202,10 @@ def forward(raw, tensors, tokens, return_layers=False, margins=None):
         if begins is not None:
             x = torch.cat([x, x0], -1) @ W["loop.in"].T + W["loop.step"][begins]
         h = layer_norm(x, W[p + "norm1"], eps)
-        y = MIXERS[layer["type"]](h + causal_conv(h, W[p + "canon1"]), W, p + "mix.", layer["mixer"], eps)
+        mixed = lambda k: h + causal_conv(h, W[f"{p}canon{k}"]) if raw.get("canon") else h
+        y = MIXERS[layer["type"]](mixed(1), W, p + "mix.", layer["mixer"], eps)
         if layer.get("mlp") is not None:
-            y = y + experts(h + causal_conv(h, W[p + "canon2"]), W, p + "mlp.", layer["mlp"], margins)
+            y = y + experts(mixed(2), W, p + "mlp.", layer["mlp"], margins)
         x = x + y
         if raw.get("token_side"):
             x = x + token_input(x, tokens, W, i, int(raw["token_side"]["dim"]), eps)
