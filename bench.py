@@ -172,7 +172,7 @@ def main():
     ap.add_argument("--perf", action="store_true",
                     help="after the timed runs, a few eager steps with the engine's timers on: average ms by kernel "
                          "class (products / attention / selection / norms / head) on stderr and under 'timers'")
-    ap.add_argument("--scenario", default="headline", choices=["headline", "small_batch64", "sparse32k", "duvulix", "gumodra", "sagedra", "nelutar"],
+    ap.add_argument("--scenario", default="headline", choices=["headline", "small_batch64", "sparse32k", "duvulix", "gumodra", "sagedra", "nelutar", "pemalorn"],
                     help="headline: the 8B shape at batch 8, context 4,096 (the default line); "
                          "small_batch64: the 0.5B shape, 64 unequal prompts through the generation loop; sparse32k: "
                          "the 8B shape with InfLLM-v2 at 32k context; duvulix: four Duvulix layers of a real model's "
@@ -183,7 +183,10 @@ def main():
                          "(differential attention, windowed attention beside a gated delta rule, four residual streams) "
                          "beside the four Gumodra layers; nelutar: four Nelutar layers of a real model's sizes (capped windowed "
                          "attention beside linear attention, windowed attention beside a delta rule with a decay a key "
-                         "channel, retention, routed experts, a layer that runs twice) beside the four Sagedra layers")
+                         "channel, retention, routed experts, a layer that runs twice) beside the four Sagedra layers; pemalorn: four Pemalorn layer "
+                         "runs of a real model's sizes (latent attention under a window, attention with rotated values "
+                         "twice, routed and identity experts, input convolutions, a token table) beside the four Duvulix "
+                         "and the four Gumodra layers")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py: this engine runs on one GPU; --gpus {args.gpus} is not supported (no multi-GPU path exists)")
@@ -619,6 +622,58 @@ def nelutar_step_bytes(raw, esize, batch, context, prefill=False):
     return weights * esize + batch * per_seq, weights
 
 
+def config_pemalorn():
+    """Three layers, the second one twice (four layer runs), of sizes that resemble a real model's: width 4,096; latent
+    attention with 32 heads of 128 + 64 features, a query latent of 1,536, a latent of 512 and a window of 2,048;
+    attention with 32 heads on 8 kv heads of 128 with rotated values; 64 experts of 1,408 and 16 identity experts, 6 a
+    token; 4 taps on what the sub-layers read; a token table of 256 numbers a layer."""
+    latent = {"heads": 32, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": 1536, "kv_rank": 512, "scale": 192 ** -0.5,
+              "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}},
+              "mask": {"size": 2048}}
+    attn = {"heads": 32, "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "rot": {"base": 500000.0, "dims": 128}}
+    moe = {"kind": "moe", "expert": {"ff": 1408}, "router": {"experts": 64, "identity": 16, "top": 6}}
+    return {
+        "architecture": "Pemalorn", "vocab": 73448, "width": 4096, "norm": {"eps": 1e-6}, "canon": {"taps": 4},
+        "token_side": {"dim": 256}, "loop": {"start": 1, "stop": 2, "times": 2},
+        "layers": [{"type": "latent_attention", "mixer": dict(latent), "mlp": moe},
+                   {"type": "attention", "mixer": dict(attn), "mlp": moe},
+                   {"type": "latent_attention", "mixer": dict(latent), "mlp": moe}],
+    }
+
+
+def pemalorn_step_bytes(raw, esize, batch, context, prefill=False):
+    """Bytes a decode step must move: every matrix that the step reads once a layer run (of a mixture: the router, and
+    an expert for every (token, choice) pair that is no identity expert, at most all of them), and per sequence what the
+    mixers read (the latent cache of the window, keys and values), the convolutions' last inputs, the token table's
+    row.  With ``prefill``: the matrix elements a prompt token is multiplied with (of a mixture: the chosen experts)."""
+    W, side, taps = raw["width"], raw["token_side"]["dim"], raw["canon"]["taps"]
+    weights = raw["vocab"] * W
+    per_seq = 0
+    loop = raw["loop"]
+    for i, layer in enumerate(raw["layers"]):
+        m = layer["mixer"]
+        w = 2 * side * W
+        s = side * esize + 2 * 4 * (taps - 1) * W
+        if layer["type"] == "latent_attention":
+            H, R, r = m["heads"], m["kv_rank"], m["rot_dim"]
+            w += (m["q_rank"] + R + r + H * m["vdim"]) * W + H * (m["dim"] + r) * m["q_rank"]
+            w += H * (m["dim"] + m["vdim"]) * R + H * m["vdim"] * W
+            s += min(context, m["mask"]["size"]) * (2 * R + r) * esize
+        else:
+            w += (m["heads"] * (m["dim"] + m["vdim"]) + m["kv_heads"] * (m["dim"] + m["vdim"]) + m["heads"]) * W
+            s += context * m["kv_heads"] * (m["dim"] + m["vdim"]) * esize
+        r = layer["mlp"]["router"]
+        real = r["experts"] / (r["experts"] + r["identity"])
+        w += (r["experts"] + r["identity"]) * W
+        pairs = r["top"] * real if prefill else min(max(batch, 1) * r["top"] * real, r["experts"])
+        w += pairs * 3 * layer["mlp"]["expert"]["ff"] * W
+        runs = loop["times"] if loop["start"] <= i < loop["stop"] else 1
+        weights += runs * w
+        per_seq += runs * s
+    weights += loop["times"] * 2 * W * W
+    return weights * esize + batch * per_seq, int(weights)
+
+
 def duvulix_scenario(args, dev):
     """Decode and prefill of the Duvulix layer shapes beside the MiniCPM4-8B layer shape (equal width, equal
     number of layers, random weights): one JSON line with both models' figures and their timers by kernel class."""
@@ -644,7 +699,14 @@ def nelutar_scenario(args, dev):
     layer_shapes_scenario(args, dev, "nelutar", "Nelutar", config_nelutar(), ("sagedra", config_sagedra()))
 
 
-def layer_shapes_scenario(args, dev, first, title, first_raw, other):
+def pemalorn_scenario(args, dev):
+    """The same for the Pemalorn layer shapes beside the Duvulix (latent attention) and the Gumodra layer shapes
+    (parallel layers with a softmax sink and routed experts): equal width, vocabulary and number of layer runs."""
+    layer_shapes_scenario(args, dev, "pemalorn", "Pemalorn", config_pemalorn(), ("duvulix", config_duvulix()),
+                          ("gumodra", config_gumodra()))
+
+
+def layer_shapes_scenario(args, dev, first, title, first_raw, *others):
     import torch
     import cpmcu_amd
     from cpmcu_amd import Engine, EngineOptions, StepEntry, ops
@@ -657,7 +719,7 @@ def layer_shapes_scenario(args, dev, first, title, first_raw, other):
     next_tok = torch.zeros(64, dtype=torch.int32, device=dev)
     read_gbs = calibrate_read(dev)
     out = {}
-    for name, raw in ((first, first_raw), other):
+    for name, raw in ((first, first_raw),) + others:
         arch = cpmcu_amd.get_architecture(raw.get("architecture") or raw["architectures"][0])
         cfg = arch.config_class.from_dict(raw)
         per_seq = -(-(args.context + args.steps + args.warmup + 64) // 64) * 64
@@ -723,6 +785,10 @@ def layer_shapes_scenario(args, dev, first, title, first_raw, other):
             step_bytes = lambda b: nelutar_step_bytes(raw, esize, b, args.context)[0]
             params = nelutar_step_bytes(raw, esize, args.batch, 0)[1]
             prefill_params = nelutar_step_bytes(raw, esize, 1, 0, prefill=True)[1]
+        elif name == "pemalorn":
+            step_bytes = lambda b: pemalorn_step_bytes(raw, esize, b, args.context)[0]
+            params = pemalorn_step_bytes(raw, esize, args.batch, 0)[1]
+            prefill_params = pemalorn_step_bytes(raw, esize, 1, 0, prefill=True)[1]
         else:
             step_bytes = lambda b: weight_bytes_per_step(cfg, esize) + b * args.context * kv_bytes_per_token(cfg, esize)
             params = weight_bytes_per_step(cfg, esize) // esize
@@ -765,7 +831,7 @@ def layer_shapes_scenario(args, dev, first, title, first_raw, other):
         "value": d["tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
         "ms_per_step": d["ms_per_step"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
         "dtype": "bf16" if esize == 2 else "fp32", "data": "synthetic",
-        "config": {"model": f"{title} layer shapes beside {other[0]} layer shapes, 4 layers each, random weights",
+        "config": {"model": f"{title} layer shapes beside {' and '.join(o[0] for o in others)} layer shapes, 4 layers each, random weights",
                    "global_batch": args.batch, "seq_len": args.context, "parallelism": "1gpu",
                    "hip_graph": bool(args.hip_graph), first: first_raw},
         "read_kernel_gbs": round(read_gbs, 1), "models": out}))
@@ -784,6 +850,9 @@ def other_scenarios(args, dev):
         return
     if args.scenario == "nelutar":
         nelutar_scenario(args, dev)
+        return
+    if args.scenario == "pemalorn":
+        pemalorn_scenario(args, dev)
         return
     import torch
     from cpmcu_amd import Engine, EngineOptions, StepEntry

@@ -461,10 +461,15 @@ __global__ __launch_bounds__(NW * TW * 64) void attention_general_mfma_kernel(
 
 // out[token][head][:] = sum_s 2^(m_s - m) o_s / sum_s 2^(m_s - m) l_s over up to 64 shares (a share without keys
 // has l = 0): lane s holds share s's (max, sum), the common maximum and the denominator are wave reductions.
+// With v_inv_freq the head is turned back by its token's position (rotated values, as head_output_kernel does for the
+// heads that no merge writes), with head_gate it is multiplied by sigmoid(head_gate[token, head]).
 __global__ void attention_general_merge_kernel(const float* __restrict__ part_o, const float2* __restrict__ part_ml,
                                                void* __restrict__ out, int out_f32, int hdv, int n_splits,
                                                const float* __restrict__ sink, int nh,
-                                               const bf16_t* __restrict__ gate, long ld_gate) {
+                                               const bf16_t* __restrict__ gate, long ld_gate,
+                                               const int* __restrict__ positions, const float* __restrict__ v_inv_freq,
+                                               int interleaved, const bf16_t* __restrict__ head_gate, long ld_head_gate) {
+    __shared__ float head[512];
     const long row = blockIdx.x;
     const float2* ml = part_ml + row * n_splits;
     const float* po = part_o + row * n_splits * hdv;
@@ -492,8 +497,30 @@ __global__ void attention_general_merge_kernel(const float* __restrict__ part_o,
             a += __int_as_float(__builtin_amdgcn_readlane(__float_as_int(wv), s)) * po[(long)s * hdv + d];
         float r = a * inv;
         if (gate) r /= 1.0f + expf(-to_f32(gate[(row / nh) * ld_gate + (row % nh) * hdv + d]));
+        if (head_gate) r /= 1.0f + expf(-to_f32(head_gate[(row / nh) * ld_head_gate + row % nh]));
+        if (v_inv_freq) {
+            head[d] = r;
+            continue;
+        }
         if (out_f32) ((float*)out)[row * hdv + d] = r;
         else ((bf16_t*)out)[row * hdv + d] = f32_to_bf16(r);
+    }
+    if (!v_inv_freq) return;
+    __syncthreads();
+    const float pos = (float)positions[row / nh];
+    const int half = hdv / 2;
+    for (int i = threadIdx.x; i < half; i += blockDim.x) {
+        const float ang = pos * v_inv_freq[i], cs = cosf(ang), sn = sinf(ang);
+        const int ia = interleaved ? 2 * i : i, ib = interleaved ? 2 * i + 1 : i + half;
+        const float u = head[ia], v2 = head[ib];
+        const float a = u * cs + v2 * sn, b = v2 * cs - u * sn;
+        if (out_f32) {
+            ((float*)out)[row * hdv + ia] = a;
+            ((float*)out)[row * hdv + ib] = b;
+        } else {
+            ((bf16_t*)out)[row * hdv + ia] = f32_to_bf16(a);
+            ((bf16_t*)out)[row * hdv + ib] = f32_to_bf16(b);
+        }
     }
 }
 
@@ -504,7 +531,12 @@ extern "C" const char* cpmcu_attention_general_mfma(const void* q, void* out, in
                                                     const int* page_table, int table_width, int page_size,
                                                     const int* positions, const int* tok_slot, int n_splits,
                                                     const int* tiles, int n_tiles, int tokens_per_tile, int v_share,
-                                                    const void* gate, long ld_gate, float softcap, hipStream_t stream) {
+                                                    const void* gate, long ld_gate, float softcap, const float* v_inv_freq,
+                                                    int interleaved, const void* head_gate, long ld_head_gate,
+                                                    hipStream_t stream) {
+    CPMCU_REQUIRE(n_splits > 1 || (!v_inv_freq && !head_gate), "attention_general_mfma: heads are turned back or gated as a whole by the merge of split keys only");
+    CPMCU_REQUIRE(!v_inv_freq || hdv % 2 == 0, "attention_general_mfma: rotated values have an even size (%d)", hdv);
+    CPMCU_REQUIRE(!head_gate || ld_head_gate >= nh, "attention_general_mfma: gate rows of %ld elements for %d heads", ld_head_gate, nh);
     CPMCU_REQUIRE(v_share >= 1 && nkv % v_share == 0, "attention_general_mfma: %d key heads do not share values in runs of %d", nkv, v_share);
     CPMCU_REQUIRE(!gate || ld_gate >= (long)nh * hdv, "attention_general_mfma: gate rows of %ld elements for %d heads of %d", ld_gate, nh, hdv);
     CPMCU_REQUIRE(n > 0 && nh > 0 && nkv > 0 && nh % nkv == 0, "attention_general_mfma: bad shape n=%d heads=%d kv_heads=%d", n, nh, nkv);
@@ -568,7 +600,8 @@ extern "C" const char* cpmcu_attention_general_mfma(const void* q, void* out, in
     if (n_splits > 1) {
         const unsigned rows = (unsigned)((long)n * nh);
         attention_general_merge_kernel<<<rows, hdv > 128 ? 256 : (hdv > 64 ? 128 : 64), 0, stream>>>(
-            part_o, (const float2*)part_ml, out, out_f32, hdv, n_splits, sink, nh, (const bf16_t*)gate, ld_gate);
+            part_o, (const float2*)part_ml, out, out_f32, hdv, n_splits, sink, nh, (const bf16_t*)gate, ld_gate,
+            positions, v_inv_freq, interleaved, (const bf16_t*)head_gate, ld_head_gate);
         CPMCU_LAUNCH_CHECK("attention_general_merge");
     }
     return nullptr;
@@ -875,7 +908,7 @@ extern "C" const char* cpmcu_latent_store(const void* qsrc, long ldq, const void
     return nullptr;
 }
 
-// What some designs put between attention and output projection, a workgroup a token: with inv_freq the values were
+// What some designs put between attention and output projection, grid (tokens, runs of heads): with inv_freq the values were
 // cached rotated by their own positions (over all dv features) and every head's sum is turned back by the query's
 // position (pairs (i, i + dv/2), or neighbours when interleaved); with gate the head is multiplied by
 // sigmoid(gate[t, head]), a number a head.  The cos and sin of a token's angles are formed once, for all its heads.
@@ -883,14 +916,16 @@ template <typename IT, typename T>
 __global__ __launch_bounds__(256) void head_output_kernel(const IT* __restrict__ o, T* __restrict__ out, int nh, int dv,
                                                           const int* __restrict__ positions,
                                                           const float* __restrict__ inv_freq, int interleaved,
-                                                          const T* __restrict__ gate, long ldg) {
+                                                          const T* __restrict__ gate, long ldg, int heads_a_run) {
     __shared__ float cs[AG_MAX_HD / 2], sn[AG_MAX_HD / 2];
     const long t = blockIdx.x;
     const int half = dv / 2;
-    const IT* src = o + t * nh * dv;
-    T* dst = out + t * nh * dv;
+    const int h0 = blockIdx.y * heads_a_run, nhr = min(heads_a_run, nh - h0);
+    const IT* src = o + (t * nh + h0) * dv;
+    T* dst = out + (t * nh + h0) * dv;
+    if (gate) gate += h0;
     if (!inv_freq) {
-        for (int i = threadIdx.x; i < nh * dv; i += 256) {
+        for (int i = threadIdx.x; i < nhr * dv; i += 256) {
             float v = to_f32(src[i]);
             if (gate) v /= 1.0f + expf(-to_f32(gate[t * ldg + i / dv]));
             dst[i] = from_f32<T>(v);
@@ -904,7 +939,7 @@ __global__ __launch_bounds__(256) void head_output_kernel(const IT* __restrict__
         sn[i] = sinf(ang);
     }
     __syncthreads();
-    for (int j = threadIdx.x; j < nh * half; j += 256) {
+    for (int j = threadIdx.x; j < nhr * half; j += 256) {
         const int h = j / half, i = j - h * half;
         const int ia = h * dv + (interleaved ? 2 * i : i), ib = h * dv + (interleaved ? 2 * i + 1 : i + half);
         const float u = to_f32(src[ia]), v = to_f32(src[ib]);
@@ -920,9 +955,13 @@ extern "C" const char* cpmcu_head_output(const void* o, int o_dtype, void* out, 
     CPMCU_REQUIRE(n > 0 && nh > 0 && dv > 0 && dv <= AG_MAX_HD, "head_output: empty shape or heads of %d (up to %d)", dv, AG_MAX_HD);
     CPMCU_REQUIRE(!inv_freq || (positions && dv % 2 == 0), "head_output: rotated values have an even size (%d)", dv);
     CPMCU_REQUIRE(!gate || ldg >= nh, "head_output: gate rows of %ld for %d heads", ldg, nh);
+    // few tokens: a workgroup takes some of a token's heads, for more workgroups
+    int run = nh;
+    while (run > 1 && (long)run * dv > 512 && (long)n * ((nh + run - 1) / run) < 512) run = (run + 1) / 2;
+    const dim3 grid(n, (nh + run - 1) / run);
 #define LAUNCH(IT, T)                                                                                              \
-    head_output_kernel<IT, T><<<n, 256, 0, stream>>>((const IT*)o, (T*)out, nh, dv, positions, inv_freq, interleaved, \
-                                                     (const T*)gate, ldg)
+    head_output_kernel<IT, T><<<grid, 256, 0, stream>>>((const IT*)o, (T*)out, nh, dv, positions, inv_freq, interleaved, \
+                                                     (const T*)gate, ldg, run)
     if (o_dtype == CPMCU_F32 && dtype == CPMCU_F32) LAUNCH(float, float);
     else if (o_dtype == CPMCU_F32 && dtype == CPMCU_BF16) LAUNCH(float, bf16_t);
     else if (o_dtype == CPMCU_BF16 && dtype == CPMCU_BF16) LAUNCH(bf16_t, bf16_t);

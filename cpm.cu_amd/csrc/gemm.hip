@@ -158,15 +158,17 @@ extern "C" const char* cpmcu_gemm_nt_heads(const void* X, long ldx, long hsx, co
 }
 
 // The product head by head in bf16 on the matrix cores (v_mfma_f32_16x16x32_bf16).  A workgroup of 4
-// wavefronts owns, for one head, 64 rows x 64 columns (WM = 4: a wavefront a tile of 16 rows) or 16 rows x 256
-// columns (WM = 1, steps of few rows: a wavefront 64 columns); a wavefront holds 4 tiles of 16 x 16 results.
+// wavefronts owns, for one head, 64 rows x 64 columns (WM = 4: a wavefront a tile of 16 rows, NT = 4 tiles of 16
+// columns) or 16 rows x 64 columns (WM = 1, steps of few rows: a wavefront 16 columns, NT = 1, so that a head's weight
+// is spread over as many wavefronts as it has strips of 16 columns).
 // Operands come straight from memory, 16 bytes a lane: lane (r, g) of a tile reads row r, columns k0 + 8g .. + 8,
 // of X and of W alike (W [N, K] row-major is the transposed operand as it lies).  K is a multiple of 8 and
-// rows start on 16-byte borders (the launcher checks).
+// rows start on 16-byte borders (the launcher checks).  No load stands in a branch: rows and columns beyond the end
+// repeat the last one (their results are not written), features beyond K read the step's first ones and are zeroed.
 typedef __bf16 hbf16x8_t __attribute__((ext_vector_type(8)));
 typedef float hfloatx4_t __attribute__((ext_vector_type(4)));
 
-template <int WM>
+template <int WM, int NT>
 __global__ __launch_bounds__(256) void gemm_heads_mfma_kernel(const bf16_t* __restrict__ X, long ldx, long hsx,
                                                               const bf16_t* __restrict__ W, bf16_t* __restrict__ Y,
                                                               long ldy, long hsy, const bf16_t* __restrict__ gate,
@@ -175,49 +177,52 @@ __global__ __launch_bounds__(256) void gemm_heads_mfma_kernel(const bf16_t* __re
     const int lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
     const int h = blockIdx.z;
     const int m0 = blockIdx.y * (WM == 4 ? 64 : 16) + (WM == 4 ? wave * 16 : 0);
-    const int n0 = blockIdx.x * (WM == 4 ? 64 : 256) + (WM == 4 ? 0 : wave * 64);
+    const int n0 = blockIdx.x * 64 + (WM == 4 ? 0 : wave * 16 * NT);
     if (m0 >= M || n0 >= N) return;
-    const bf16_t* xp = X + (long)h * hsx + (long)min(m0 + r, M - 1) * ldx + g * 8;
-    const bf16_t* wp = W + (long)h * N * K + g * 8;
-    const bool row_ok = m0 + r < M;
-    hfloatx4_t acc[4];
+    const bf16_t* xp = X + (long)h * hsx + (long)min(m0 + r, M - 1) * ldx;
+    const bf16_t* wp = W + (long)h * N * K;
+    hfloatx4_t acc[NT];
+    long wrow[NT];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) acc[j] = hfloatx4_t{0.f, 0.f, 0.f, 0.f};
-    long wrow[4];
-    bool col_ok[4];
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-        col_ok[j] = n0 + 16 * j + r < N;
+    for (int j = 0; j < NT; ++j) {
+        acc[j] = hfloatx4_t{0.f, 0.f, 0.f, 0.f};
         wrow[j] = (long)min(n0 + 16 * j + r, N - 1) * K;
     }
-#pragma unroll 2
+    // the gate's numbers of this lane's results are asked for before the product's operands
+    float gs[4][NT];
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < NT; ++j) {
+            gs[i][j] = 0.f;
+            if (gate) {
+                const long m = min(m0 + 4 * g + i, M - 1);
+                gs[i][j] = to_f32(gate[m * ldg + (gate_wide ? (long)h * N + min(n0 + 16 * j + r, N - 1) : h)]);
+            }
+        }
+    const hbf16x8_t zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll (NT == 1 ? 8 : 2)
     for (int k0 = 0; k0 < K; k0 += 32) {
         const bool k_ok = k0 + g * 8 < K;
-        hbf16x8_t a = {0, 0, 0, 0, 0, 0, 0, 0};
-        if (k_ok && row_ok) a = *(const hbf16x8_t*)(xp + k0);
-        hbf16x8_t b[4];
+        const int kk = k0 + (k_ok ? g * 8 : 0);
+        hbf16x8_t a = *(const hbf16x8_t*)(xp + kk);
+        a = k_ok ? a : zero8;
+        hbf16x8_t b[NT];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-            b[j] = hbf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
-            if (k_ok && col_ok[j]) b[j] = *(const hbf16x8_t*)(wp + wrow[j] + k0);
-        }
+        for (int j = 0; j < NT; ++j) b[j] = *(const hbf16x8_t*)(wp + wrow[j] + kk);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b[j], acc[j], 0, 0, 0);
+        for (int j = 0; j < NT; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, k_ok ? b[j] : zero8, acc[j], 0, 0, 0);
     }
     // lane (column r, g): acc[j][i] is the result of row m0 + 4g + i, column n0 + 16j + r
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
         const int m = m0 + 4 * g + i;
         if (m >= M) continue;
-        float gs = 1.f;
-        if (gate && !gate_wide) gs = 1.0f / (1.0f + expf(-to_f32(gate[(long)m * ldg + h])));
         bf16_t* yr = Y + (long)h * hsy + (long)m * ldy;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
+        for (int j = 0; j < NT; ++j) {
             const int n = n0 + 16 * j + r;
-            if (n >= N) continue;
-            if (gate_wide) gs = 1.0f / (1.0f + expf(-to_f32(gate[(long)m * ldg + (long)h * N + n])));
-            yr[n] = f32_to_bf16(gs * acc[j][i]);
+            if (n < N) yr[n] = f32_to_bf16(gate ? acc[j][i] / (1.0f + expf(-gs[i][j])) : acc[j][i]);
         }
     }
 }
@@ -233,14 +238,14 @@ extern "C" const char* cpmcu_gemm_nt_heads_mfma(const void* X, long ldx, long hs
                   "gemm_heads_mfma: rows of %ld / %ld elements cannot hold %d heads", ldx, ldy, H);
     CPMCU_REQUIRE(H <= 65535, "gemm_heads_mfma: %d heads exceed the launch grid", H);
     if (M <= 16) {
-        dim3 grid((N + 255) / 256, 1, H);
-        gemm_heads_mfma_kernel<1><<<grid, 256, 0, stream>>>((const bf16_t*)X, ldx, hsx, (const bf16_t*)W, (bf16_t*)Y, ldy,
-                                                            hsy, (const bf16_t*)gate, ldg, gate && gate_wide, M, N, K);
+        dim3 grid((N + 63) / 64, 1, H);
+        gemm_heads_mfma_kernel<1, 1><<<grid, 256, 0, stream>>>((const bf16_t*)X, ldx, hsx, (const bf16_t*)W, (bf16_t*)Y, ldy,
+                                                               hsy, (const bf16_t*)gate, ldg, gate && gate_wide, M, N, K);
     } else {
         dim3 grid((N + 63) / 64, (M + 63) / 64, H);
         CPMCU_REQUIRE(grid.y <= 65535, "gemm_heads_mfma: M=%d too large for one launch", M);
-        gemm_heads_mfma_kernel<4><<<grid, 256, 0, stream>>>((const bf16_t*)X, ldx, hsx, (const bf16_t*)W, (bf16_t*)Y, ldy,
-                                                            hsy, (const bf16_t*)gate, ldg, gate && gate_wide, M, N, K);
+        gemm_heads_mfma_kernel<4, 4><<<grid, 256, 0, stream>>>((const bf16_t*)X, ldx, hsx, (const bf16_t*)W, (bf16_t*)Y, ldy,
+                                                               hsy, (const bf16_t*)gate, ldg, gate && gate_wide, M, N, K);
     }
     CPMCU_LAUNCH_CHECK("gemm_nt_heads_mfma");
     return nullptr;

@@ -12,7 +12,10 @@
 //  * moe_gated_kernel: act[t, k, :] = act(Wg_e h_t) * (Wu_e h_t) for the k-th chosen expert e of token t (the
 //    nonlinearities of common.h: SiLU, or the clamped swish with its limit); the experts' gate and up rows are
 //    stacked: wgu [E, 2F, H], gate rows first.
-//  * moe_down_kernel: out[t] = sum_k w[t, k] Wd_e act[t, k] (+ sg[t] * shared[t]); wd [E, H, F]; float out.
+//  * moe_down_kernel: out[t] = sum_k w[t, k] Wd_e act[t, k] (+ sg[t] * shared[t]); wd [E, H, F]; float out.  With a
+//    residual (Join) the layer's sum ends here: x[t] += out[t] + another result of the layer (float partial sums or
+//    one bf16 / float tensor, and a bias), in place, and x once more in the activations' type for a product that
+//    reads it; nothing else is written.
 //
 // A wavefront owns output rows and its lanes stride over the input features (16-byte loads when the rows are
 // aligned), so an expert's weights stream once for every token that chose it: the form for steps of few tokens.
@@ -21,6 +24,20 @@
 #define MOE_MAX_EXPERTS 1024
 enum { MOE_SCORE_SOFTMAX = 0, MOE_SCORE_SIGMOID = 1 };
 enum { MOE_GROUP_MAX = 0, MOE_GROUP_TOP2_SUM = 1 };
+
+// Where a layer's sum ends: the residual x [n, H], another result `a` to add (parts `stride` apart; may be absent) with
+// an optional bias, and a copy of the new x in the activations' type (may be absent)
+struct Join {
+    float* x;
+    const void* a;
+    int a_bf16, a_parts;
+    long a_stride;
+    const float* a_bias;
+    void* copy;
+};
+__device__ inline float join_part(const Join& j, int p, long i) {
+    return j.a_bf16 ? to_f32(((const bf16_t*)j.a)[p * j.a_stride + i]) : ((const float*)j.a)[p * j.a_stride + i];
+}
 
 template <typename T> struct Vec8;
 template <> struct Vec8<bf16_t> { typedef uint4 type; };
@@ -179,7 +196,8 @@ __global__ __launch_bounds__(64) void moe_select_kernel(const float* __restrict_
 extern "C" const char* cpmcu_moe_route(const void* h, long ldh, int dtype, const float* wr, const float* correction,
                                        const float* w_sg, int n, int H, int E, int n_groups, int keep_groups, int top,
                                        float* logits, int* idx_out, float* w_out, float* sg_out, int score_fn,
-                                       int group_fn, float weight_scale, int normalize, hipStream_t stream) {
+                                       int group_fn, float weight_scale, int normalize, int logits_ready,
+                                       hipStream_t stream) {
     CPMCU_REQUIRE((score_fn == MOE_SCORE_SOFTMAX || score_fn == MOE_SCORE_SIGMOID) &&
                   (group_fn == MOE_GROUP_MAX || group_fn == MOE_GROUP_TOP2_SUM),
                   "moe_route: unknown score function %d or group score %d", score_fn, group_fn);
@@ -191,7 +209,9 @@ extern "C" const char* cpmcu_moe_route(const void* h, long ldh, int dtype, const
                   top, keep_groups * (E / n_groups));
     CPMCU_REQUIRE(!w_sg || sg_out, "moe_route: a place for the shared gate is missing");
     dim3 grid(n, (E + 1 + 3) / 4);
-    if (dtype == CPMCU_F32)
+    if (logits_ready) {
+        // the rows of logits come from a product of the caller's
+    } else if (dtype == CPMCU_F32)
         moe_logits_kernel<float><<<grid, 256, 0, stream>>>((const float*)h, ldh, wr, w_sg, H, E, logits);
     else if (dtype == CPMCU_BF16)
         moe_logits_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)h, ldh, wr, w_sg, H, E, logits);
@@ -204,7 +224,7 @@ extern "C" const char* cpmcu_moe_route(const void* h, long ldh, int dtype, const
     return nullptr;
 }
 
-#define MOE_ROWS 4       // output rows a wavefront
+#define MOE_ROWS 4       // output rows a wavefront (moe_down_kernel names its four)
 
 // grid (tokens * top, ceil(F / 16)), 256 threads: wavefront w takes rows [16 y + 4 w, +4) of the expert's F
 template <typename T>
@@ -249,56 +269,116 @@ extern "C" const char* cpmcu_moe_gated(const void* h, long ldh, int dtype, const
     return nullptr;
 }
 
-// grid (tokens, ceil(H / 16)), 256 threads.  shared: the every-token expert's output [n, H] (or float partial
+// grid (tokens, ceil(H / 16)), 256 threads: a wavefront owns 4 columns and reads their 4 weight rows of a chosen expert
+// together, against one piece of the pair's act row.  shared: the every-token expert's output [n, H] (or float partial
 // sums [parts][n][H]), multiplied by sg[t]; may be absent.  h: the experts' input, what identity experts (e >= E) add.
+// What the end adds (shared, residual, the layer's other result) is asked for first: 16 lanes a column bring it, a part a
+// lane.
 template <typename T, typename ST>
 __global__ __launch_bounds__(256) void moe_down_kernel(const T* __restrict__ act, const T* __restrict__ wd,
                                                        const int* __restrict__ idx, const float* __restrict__ w,
                                                        const ST* __restrict__ shared, int shared_parts,
                                                        long shared_stride, const float* __restrict__ sg,
                                                        const T* __restrict__ h, long ldh, int E,
-                                                       float* __restrict__ out, int H, int F, int top) {
+                                                       float* __restrict__ out, int H, int F, int top, Join join) {
     const long t = blockIdx.x;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const bool vec = (F % 8 == 0) && ((uintptr_t)act % 32 == 0) && ((uintptr_t)wd % 32 == 0);
     const int c0 = blockIdx.y * 4 * MOE_ROWS + wave * MOE_ROWS;
-#pragma unroll
-    for (int r = 0; r < MOE_ROWS; ++r) {
-        const int c = c0 + r;
-        if (c >= H) break;
-        float s = 0.f, same = 0.f;
-        for (int k = 0; k < top; ++k) {
-            const int e = idx[t * top + k];
-            if (e >= E) {
-                same += w[t * top + k];
-                continue;
-            }
-            s += w[t * top + k] * lane_dot<T, T>(wd + ((long)e * H + c) * F, act + (t * top + k) * F, F, lane, vec);
+    if (c0 >= H) return;
+    const int mine = c0 + (lane >> 4), p0 = lane & 15;               // this lane's column at the end, and its part
+    const long at = t * H + min(mine, H - 1);
+    float extra = 0.f;
+    if (shared) {
+        for (int p = p0; p < shared_parts; p += 16) extra += to_f32(shared[(long)p * shared_stride + at]);
+        if (sg) extra *= sg[t];
+    }
+    if (join.x) {
+        for (int p = p0; p < join.a_parts; p += 16) extra += join_part(join, p, at);
+        if (p0 == 15) extra += join.x[at] + (join.a_bias ? join.a_bias[min(mine, H - 1)] : 0.f);
+    }
+    const long row0 = (long)min(c0, H - 1) * F, row1 = (long)min(c0 + 1, H - 1) * F, row2 = (long)min(c0 + 2, H - 1) * F,
+               row3 = (long)min(c0 + 3, H - 1) * F;
+    float s0 = 0.f, s1 = 0.f, s2 = 0.f, s3 = 0.f, same = 0.f;
+    for (int k = 0; k < top; ++k) {
+        const int e = idx[t * top + k];
+        const float wk = w[t * top + k];
+        if (e >= E) {
+            same += wk;
+            continue;
         }
-        s = wave_sum(s);
-        if (lane == 0) {
-            if (h && same != 0.f) s += same * to_f32(h[t * ldh + c]);
-            if (shared) {
-                float v = 0.f;
-                for (int p = 0; p < shared_parts; ++p) v += to_f32(shared[(long)p * shared_stride + t * H + c]);
-                s += (sg ? sg[t] : 1.0f) * v;
+        const T* ap = act + (t * top + k) * F;
+        const T* wp = wd + (long)e * H * F;
+        float d0 = 0.f, d1 = 0.f, d2 = 0.f, d3 = 0.f;
+        if (vec) {
+            for (int c = lane * 8; c < F; c += 64 * 8) {
+                float x[8], y0[8], y1[8], y2[8], y3[8];
+                load8<T>(wp + row0 + c, y0);
+                load8<T>(wp + row1 + c, y1);
+                load8<T>(wp + row2 + c, y2);
+                load8<T>(wp + row3 + c, y3);
+                load8<T>(ap + c, x);
+#pragma unroll
+                for (int i = 0; i < 8; ++i) {
+                    d0 += x[i] * y0[i];
+                    d1 += x[i] * y1[i];
+                    d2 += x[i] * y2[i];
+                    d3 += x[i] * y3[i];
+                }
             }
-            out[t * H + c] = s;
+        } else {
+            for (int c = lane; c < F; c += 64) {
+                const float x = to_f32(ap[c]);
+                d0 += x * to_f32(wp[row0 + c]);
+                d1 += x * to_f32(wp[row1 + c]);
+                d2 += x * to_f32(wp[row2 + c]);
+                d3 += x * to_f32(wp[row3 + c]);
+            }
+        }
+        s0 += wk * d0;
+        s1 += wk * d1;
+        s2 += wk * d2;
+        s3 += wk * d3;
+    }
+    s0 = wave_sum(s0);
+    s1 = wave_sum(s1);
+    s2 = wave_sum(s2);
+    s3 = wave_sum(s3);
+    extra = row16_sum(extra);                       // the 16 lanes of a column are one row of lanes
+    const int r = lane >> 4;
+    float v = (r == 0 ? s0 : (r == 1 ? s1 : (r == 2 ? s2 : s3))) + extra;
+    if (p0 == 0 && mine < H) {
+        if (h && same != 0.f) v += same * to_f32(h[t * ldh + mine]);
+        if (join.x) {
+            join.x[at] = v;
+            if (join.copy) ((T*)join.copy)[at] = from_f32<T>(v);
+        } else {
+            out[at] = v;
         }
     }
+}
+
+static const char* join_check(const Join& j, const float* out) {
+    CPMCU_REQUIRE(j.x || out, "experts: nowhere to write");
+    CPMCU_REQUIRE(!j.x || (j.a_parts >= 0 && j.a_parts <= 32 && (j.a != nullptr) == (j.a_parts > 0)),
+                  "experts: %d parts of the layer's other result (up to 32 are taken)", j.a_parts);
+    return nullptr;
 }
 
 extern "C" const char* cpmcu_moe_down(const void* act, int dtype, const void* wd, const int* idx, const float* w,
                                       const void* shared, int shared_dtype, int shared_parts, long shared_stride,
                                       const float* sg, const void* h, long ldh, int E, float* out, int n, int H, int F,
-                                      int top, hipStream_t stream) {
+                                      int top, float* x, const void* a, int a_dtype, int a_parts, long a_stride,
+                                      const float* a_bias, void* copy, hipStream_t stream) {
+    const Join join{x, a, a_dtype == CPMCU_BF16, a ? a_parts : 0, a_stride, a_bias, copy};
+    if (const char* m = join_check(join, out)) return m;
     CPMCU_REQUIRE(n > 0 && H > 0 && F > 0 && top > 0 && E > 0, "moe_down: empty shape");
     const int hy = (H + 4 * MOE_ROWS - 1) / (4 * MOE_ROWS);
     CPMCU_REQUIRE(hy <= 65535, "moe_down: a width of %d exceeds the launch grid", H);
     dim3 grid(n, hy);
 #define LAUNCH(Tv, STv)                                                                                            \
     moe_down_kernel<Tv, STv><<<grid, 256, 0, stream>>>((const Tv*)act, (const Tv*)wd, idx, w, (const STv*)shared,   \
-                                                       shared_parts, shared_stride, sg, (const Tv*)h, ldh, E, out, H, F, top)
+                                                       shared_parts, shared_stride, sg, (const Tv*)h, ldh, E, out, H, F, top, join)
     const int sd = shared ? shared_dtype : CPMCU_F32;
     if (dtype == CPMCU_F32 && sd == CPMCU_F32) LAUNCH(float, float);
     else if (dtype == CPMCU_BF16 && sd == CPMCU_F32) LAUNCH(bf16_t, float);
@@ -485,24 +565,54 @@ __global__ __launch_bounds__(256) void moe_down_mfma_kernel(const bf16_t* __rest
         }
 }
 
-template <typename ST>
+// V neighbouring columns a thread (4: 8-byte loads of a pair's row)
+template <typename ST, int V>
 __global__ __launch_bounds__(256) void moe_combine_kernel(const bf16_t* __restrict__ y, const float* __restrict__ w,
                                                           const ST* __restrict__ shared, int shared_parts,
                                                           long shared_stride, const float* __restrict__ sg,
                                                           const int* __restrict__ idx, const bf16_t* __restrict__ h, long ldh,
-                                                          int E, float* __restrict__ out, long total, int H, int top) {
-    for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < total; i += (long)gridDim.x * 256) {
+                                                          int E, float* __restrict__ out, long total, int H, int top, Join join) {
+    auto load = [](const bf16_t* p, float* v) {
+        if (V == 4) {
+            const uint2 u = *(const uint2*)p;
+            v[0] = __uint_as_float(u.x << 16); v[1 % V] = __uint_as_float(u.x & 0xffff0000u);
+            v[2 % V] = __uint_as_float(u.y << 16); v[3 % V] = __uint_as_float(u.y & 0xffff0000u);
+        } else {
+            v[0] = to_f32(*p);
+        }
+    };
+    for (long i = V * ((long)blockIdx.x * 256 + threadIdx.x); i < total; i += V * (long)gridDim.x * 256) {
         const long t = i / H;
         const int c = (int)(i - t * H);
-        float s = 0.f;
-        for (int k = 0; k < top; ++k)
-            s += w[t * top + k] * to_f32(idx[t * top + k] < E ? y[(t * top + k) * H + c] : h[t * ldh + c]);
-        if (shared) {
-            float v = 0.f;
-            for (int p = 0; p < shared_parts; ++p) v += to_f32(shared[(long)p * shared_stride + i]);
-            s += (sg ? sg[t] : 1.0f) * v;
+        float s[V];
+#pragma unroll
+        for (int e = 0; e < V; ++e) s[e] = 0.f;
+#pragma unroll 2
+        for (int k = 0; k < top; ++k) {
+            float v[V];
+            load(idx[t * top + k] < E ? y + (t * top + k) * H + c : h + t * ldh + c, v);
+#pragma unroll
+            for (int e = 0; e < V; ++e) s[e] += w[t * top + k] * v[e];
         }
-        out[i] = s;
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+            if (shared) {
+                float v = 0.f;
+                for (int p = 0; p < shared_parts; ++p) v += to_f32(shared[(long)p * shared_stride + i + e]);
+                s[e] += (sg ? sg[t] : 1.0f) * v;
+            }
+            if (join.x) {
+                s[e] += join.x[i + e] + (join.a_bias ? join.a_bias[c + e] : 0.f);
+                for (int p = 0; p < join.a_parts; ++p) s[e] += join_part(join, p, i + e);
+            }
+        }
+        float* dst = join.x ? join.x : out;
+        if (V == 4) *(float4*)(dst + i) = make_float4(s[0], s[1 % V], s[2 % V], s[3 % V]);
+        else dst[i] = s[0];
+        if (join.copy) {
+#pragma unroll
+            for (int e = 0; e < V; ++e) ((bf16_t*)join.copy)[i + e] = f32_to_bf16(s[e]);
+        }
     }
 }
 
@@ -512,7 +622,11 @@ extern "C" const char* cpmcu_moe_experts_mfma(const void* h, long ldh, const voi
                                               const float* w, const void* shared, int shared_dtype, int shared_parts,
                                               long shared_stride, const float* sg, void* act, void* y, int* rows,
                                               int* tile_expert, int* n_tiles, int max_tiles, float* out, int n, int H,
-                                              int F, int E, int top, int act_fn, float act_limit, hipStream_t stream) {
+                                              int F, int E, int top, int act_fn, float act_limit, float* x, const void* a,
+                                              int a_dtype, int a_parts, long a_stride, const float* a_bias, void* copy,
+                                              hipStream_t stream) {
+    const Join join{x, a, a_dtype == CPMCU_BF16, a ? a_parts : 0, a_stride, a_bias, copy};
+    if (const char* m = join_check(join, out)) return m;
     CPMCU_REQUIRE(n > 0 && H > 0 && F > 0 && E > 0 && top > 0, "moe_experts_mfma: empty shape");
     CPMCU_REQUIRE(CPMCU_ACT_KNOWN(act_fn), "moe_experts_mfma: unknown nonlinearity %d", act_fn);
     CPMCU_REQUIRE(E <= MOE_MAX_EXPERTS, "moe_experts_mfma: %d experts (up to %d are taken)", E, MOE_MAX_EXPERTS);
@@ -531,13 +645,21 @@ extern "C" const char* cpmcu_moe_experts_mfma(const void* h, long ldh, const voi
                                                                            tile_expert, n_tiles, (bf16_t*)y, H, F);
     CPMCU_LAUNCH_CHECK("moe_down_mfma");
     const long total = (long)n * H;
-    const int blocks = (int)((total + 255) / 256 < 8192 ? (total + 255) / 256 : 8192);
-    if (!shared || shared_dtype == CPMCU_F32)
-        moe_combine_kernel<float><<<blocks, 256, 0, stream>>>((const bf16_t*)y, w, (const float*)shared, shared_parts,
-                                                              shared_stride, sg, idx, (const bf16_t*)h, ldh, E, out, total, H, top);
-    else
-        moe_combine_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)y, w, (const bf16_t*)shared, shared_parts,
-                                                               shared_stride, sg, idx, (const bf16_t*)h, ldh, E, out, total, H, top);
+    const bool vec = H % 4 == 0 && ldh % 4 == 0 && (uintptr_t)y % 16 == 0 && (uintptr_t)(x ? x : out) % 16 == 0;
+    const long work = vec ? total / 4 : total;
+    const int blocks = (int)((work + 255) / 256 < 8192 ? (work + 255) / 256 : 8192);
+#define COMBINE(STv, Vv)                                                                                              \
+    moe_combine_kernel<STv, Vv><<<blocks, 256, 0, stream>>>((const bf16_t*)y, w, (const STv*)shared, shared_parts,   \
+                                                            shared_stride, sg, idx, (const bf16_t*)h, ldh, E, out,  \
+                                                            total, H, top, join)
+    if (!shared || shared_dtype == CPMCU_F32) {
+        if (vec) COMBINE(float, 4);
+        else COMBINE(float, 1);
+    } else {
+        if (vec) COMBINE(bf16_t, 4);
+        else COMBINE(bf16_t, 1);
+    }
+#undef COMBINE
     CPMCU_LAUNCH_CHECK("moe_combine");
     return nullptr;
 }

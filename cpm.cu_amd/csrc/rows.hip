@@ -13,7 +13,8 @@
 //    conv_rows_remember_kernel then moves the slots on to the step's last inputs.
 //  * add_rows_kernel: x += A + F (partial sums and biases), and x again in the activations' element type: what a
 //    product that reads the residual itself takes.
-//  * gated_lookup_kernel: g[t, j] = act(z[t, j]) * table[id_t, off + j].
+//  * gated_lookup_kernel: g[t, j] = act(z[t, j]) * table[id_t, off + j]; lookup_strip_kernel does the product z = x W^T
+//    as well, for decode steps of at most 16 tokens in bf16.
 #include "common.h"
 #include "vec4.h"
 
@@ -412,5 +413,79 @@ extern "C" const char* cpmcu_gated_lookup(const void* z, int z_dtype, int parts,
     else CPMCU_FAIL("gated_lookup: unsupported dtypes z=%d table=%d", z_dtype, dtype);
 #undef LAUNCH
     CPMCU_LAUNCH_CHECK("gated_lookup");
+    return nullptr;
+}
+
+// The product and the lookup of a decode step in one launch: a workgroup owns a strip of 16 columns over all of K, its NW
+// wavefronts take a contiguous share of the 128-column blocks each (weight tiled as for the other strip kernels: [strip
+// of 16 rows][128-column block][i][lane][8], zero padded), add up through LDS, and the first one finishes.
+typedef __bf16 rbf16x8_t __attribute__((ext_vector_type(8)));
+typedef float rfloatx4_t __attribute__((ext_vector_type(4)));
+
+template <int PF, int NW>
+__global__ __launch_bounds__(NW * 64) void lookup_strip_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ W, int M,
+                                                               int D, int K, const bf16_t* __restrict__ table, long ld_table,
+                                                               long off, const int* __restrict__ ids,
+                                                               bf16_t* __restrict__ out, int act) {
+    __shared__ float red[NW - 1][4][64];
+    const int strip = blockIdx.x;
+    const int wave = __builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));
+    const int lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
+    const int nkb = (K + 127) / 128, per_wave = (nkb + NW - 1) / NW;
+    const int kb0 = wave * per_wave, kb1 = min(kb0 + per_wave, nkb);
+    const bf16_t* wp = W + (long)strip * nkb * 2048 + lane * 8;
+    const bf16_t* ap = A + (long)min(r, M - 1) * K;             // rows beyond the step repeat its last token
+    const int col = strip * 16 + 4 * g;
+    // what the end needs is asked for first: the table's numbers of this lane's token and columns
+    float e[4];
+    const bf16_t* tp = table + (long)ids[min(r, M - 1)] * ld_table + off;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) e[i] = to_f32(tp[min(col + i, D - 1)]);
+    rfloatx4_t acc = {0.f, 0.f, 0.f, 0.f};
+    for (int kb = kb0; kb < kb1; kb += PF) {
+        // a block beyond the wavefront's last repeats the matrix's last and is not multiplied; columns beyond K repeat
+        // the row's last 8 and meet the weight's zero padding
+        rbf16x8_t wv[PF][4], av[PF][4];
+#pragma unroll
+        for (int j = 0; j < PF; ++j) {
+            const int kbc = min(kb + j, nkb - 1);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                wv[j][i] = *(const rbf16x8_t*)(wp + ((long)kbc * 4 + i) * 512);
+                av[j][i] = *(const rbf16x8_t*)(ap + min(kbc * 128 + i * 32 + g * 8, K - 8));
+            }
+        }
+#pragma unroll
+        for (int j = 0; j < PF; ++j)
+            if (kb + j < kb1) {
+#pragma unroll
+                for (int i = 0; i < 4; ++i) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[j][i], av[j][i], acc, 0, 0, 0);
+            }
+    }
+    if (wave > 0) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) red[wave - 1][i][lane] = acc[i];
+    }
+    __syncthreads();
+    if (wave > 0 || r >= M) return;
+    // lane (token r, g): acc[i] is column 16 * strip + 4g + i
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        float z = acc[i];
+#pragma unroll
+        for (int w = 0; w < NW - 1; ++w) z += red[w][i][lane];
+        if (col + i < D) out[(long)r * D + col + i] = f32_to_bf16(gate_act(z, act) * e[i]);
+    }
+}
+
+extern "C" const char* cpmcu_lookup_strip(const void* A, const void* W, int M, int D, int K, const void* table, long ld_table,
+                                          long off, const int* ids, void* out, int act, hipStream_t stream) {
+    CPMCU_REQUIRE(M > 0 && M <= 16, "lookup_strip: %d tokens (1..16 are taken)", M);
+    CPMCU_REQUIRE(D > 0 && K > 0 && K % 8 == 0 && off >= 0 && off + D <= ld_table, "lookup_strip: %d columns, K=%d (a multiple of 8)", D, K);
+    CPMCU_REQUIRE(A && W && table && ids && out && (uintptr_t)A % 16 == 0 && (uintptr_t)W % 16 == 0, "lookup_strip: operands must be 16-byte aligned");
+    CPMCU_REQUIRE(act == CPMCU_ACT_SILU || act == CPMCU_ACT_GELU_TANH, "lookup_strip: unknown nonlinearity %d", act);
+    lookup_strip_kernel<4, 8><<<(D + 15) / 16, 512, 0, stream>>>((const bf16_t*)A, (const bf16_t*)W, M, D, K, (const bf16_t*)table,
+                                                               ld_table, off, ids, (bf16_t*)out, act);
+    CPMCU_LAUNCH_CHECK("lookup_strip");
     return nullptr;
 }

@@ -1044,6 +1044,26 @@ def gated_lookup(z: torch.Tensor, table: torch.Tensor, offset: int, ids: torch.T
                                              c_int(n), c_int(D), c_int(GATE_ACTIVATIONS[activation]), _stream()))
 
 
+LOOKUP_STRIP_ROWS = 16
+
+
+def lookup_strip(x: torch.Tensor, w: "TiledWeight", table: torch.Tensor, offset: int, ids: torch.Tensor, out: torch.Tensor,
+                 activation: str = "gelu_tanh"):
+    """gated_lookup of z = x . w^T in one launch, for a step of at most 16 tokens: x bfloat16 [n, K], w tiled [D, K]."""
+    _need(x, "lookup x", torch.bfloat16, (None, None))
+    n, K = x.shape
+    if not isinstance(w, TiledWeight) or w.K != K:
+        raise KernelError(f"lookup_strip: the weight must be tiled for K = {K}")
+    _need(out, "lookup out", torch.bfloat16, (n, w.N))
+    _need(table, "lookup table", torch.bfloat16, (None, None))
+    if offset < 0 or offset + w.N > table.shape[1]:
+        raise KernelError(f"lookup_strip: columns {offset}..{offset + w.N} of a table of {table.shape[1]}")
+    _need(ids, "lookup ids", torch.int32, (n,))
+    _check(_fn("rows", "cpmcu_lookup_strip")(_p(x), _p(w.data), c_int(n), c_int(w.N), c_int(K), _p(table),
+                                             c_long(table.shape[1]), c_long(offset), _p(ids), _p(out),
+                                             c_int(GATE_ACTIVATIONS[activation]), _stream()))
+
+
 def pair_norm_mean(a: torch.Tensor, a_bias: Optional[torch.Tensor], b: torch.Tensor, b_bias: Optional[torch.Tensor],
                    wa: torch.Tensor, wb: torch.Tensor, eps: float, out: torch.Tensor):
     """out = (a / rms(a) * wa + b / rms(b) * wb) / 2 row by row in float, rms(v) = sqrt(mean(v^2) + eps): the
@@ -1207,7 +1227,8 @@ MOE_GROUP_SCORES = {"max": 0, "top2_sum": 1}
 def moe_route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.Tensor], shared_gate: Optional[torch.Tensor],
               n_groups: int, keep_groups: int, top: int, idx: torch.Tensor, weights: torch.Tensor,
               shared_out: Optional[torch.Tensor] = None, logits: Optional[torch.Tensor] = None,
-              score: str = "softmax", group_score: str = "max", weight_scale: float = 1.0, normalize: bool = True):
+              score: str = "softmax", group_score: str = "max", weight_scale: float = 1.0, normalize: bool = True,
+              logits_ready: bool = False):
     """Routing of every token to ``top`` of E experts.  Logits router . h in float (router float32 [E, H]), scores
     s = softmax over the experts (``score`` 'sigmoid': of each logit alone); choice scores s + correction; the
     experts form n_groups equal groups of neighbours, of which only the keep_groups with the largest group score may
@@ -1215,7 +1236,10 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.
     largest choice scores win (ties: the lower index); weights = s of the chosen / (their sum + 1e-20) *
     weight_scale (without ``normalize`` s * weight_scale).  idx int32 [n, top], weights float32 [n, top].
     shared_gate (float32 [H]): shared_out[t] = sigmoid(shared_gate . h[t]).  logits: float32 [n, E + 1] of scratch
-    (allocated here when absent: a caller that must not allocate brings it)."""
+    (allocated here when absent: a caller that must not allocate brings it); with logits_ready it holds the products
+    (the shared gate's in column E) already."""
+    if logits_ready and logits is None:
+        raise KernelError("moe_route: the logits are missing")
     ldh = _ld(h, "router input")
     n, H = h.shape
     _need(router, "router weight", torch.float32, (None, H))
@@ -1236,7 +1260,8 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.
     _check(_fn("moe", "cpmcu_moe_route")(_p(h), c_long(ldh), c_int(_code(h)), _p(router), _p(correction), _p(shared_gate),
                                          c_int(n), c_int(H), c_int(E), c_int(n_groups), c_int(keep_groups), c_int(top),
                                          _p(logits), _p(idx), _p(weights), _p(shared_out), c_int(MOE_SCORES[score]),
-                                         c_int(MOE_GROUP_SCORES[group_score]), c_float(weight_scale), c_int(1 if normalize else 0), _stream()))
+                                         c_int(MOE_GROUP_SCORES[group_score]), c_float(weight_scale), c_int(1 if normalize else 0),
+                                         c_int(1 if logits_ready else 0), _stream()))
 
 
 def moe_gated(h: torch.Tensor, gate_up: torch.Tensor, idx: torch.Tensor, act: torch.Tensor, activation="silu"):
@@ -1256,12 +1281,42 @@ def moe_gated(h: torch.Tensor, gate_up: torch.Tensor, idx: torch.Tensor, act: to
                                          c_int(H), c_int(F2 // 2), c_int(top), c_int(E), *_act(activation), _stream()))
 
 
-def moe_down(act: torch.Tensor, down: torch.Tensor, idx: torch.Tensor, weights: torch.Tensor, out: torch.Tensor,
+class Join:
+    """Where a layer's sum ends: x float32 [n, H] += the experts' result + another result ``a`` of the layer ([n, H] or
+    float partial sums [P, n, H]; may be None) + ``a_bias`` (float32 [H] or None), in place; ``copy`` (may be None): the
+    new x in the activations' type."""
+    __slots__ = ("x", "a", "a_bias", "copy")
+
+    def __init__(self, x: torch.Tensor, a: Optional[torch.Tensor] = None, a_bias: Optional[torch.Tensor] = None,
+                 copy: Optional[torch.Tensor] = None):
+        self.x, self.a, self.a_bias, self.copy = x, a, a_bias, copy
+
+
+JOIN_MAX_PARTS = 32
+
+
+def _join_args(join: Optional[Join], n: int, H: int, dtype: torch.dtype):
+    if join is None:
+        return (_p(None), _p(None), c_int(F32), c_int(0), c_long(0), _p(None), _p(None))
+    _need(join.x, "experts residual", torch.float32, (n, H))
+    parts = stride = 0
+    if join.a is not None:
+        parts, stride = _parts_of(join.a, n, H, "experts other result")
+    if join.a_bias is not None:
+        _need(join.a_bias, "experts other bias", torch.float32, (H,))
+    if join.copy is not None:
+        _need(join.copy, "experts residual copy", dtype, (n, H))
+    return (_p(join.x), _p(join.a), c_int(_code(join.a) if join.a is not None else F32), c_int(parts), c_long(stride),
+            _p(join.a_bias), _p(join.copy))
+
+
+def moe_down(act: torch.Tensor, down: torch.Tensor, idx: torch.Tensor, weights: torch.Tensor, out: Optional[torch.Tensor],
              shared: Optional[torch.Tensor] = None, shared_gate: Optional[torch.Tensor] = None,
-             h: Optional[torch.Tensor] = None):
+             h: Optional[torch.Tensor] = None, join: Optional[Join] = None):
     """out[t] = sum_k weights[t, k] * Wd_e act[t, k] (+ shared_gate[t] * shared[t]); down [E, H, F]; out float32
     [n, H]; shared [n, H] or float partial sums [P, n, H].  h [n, H]: the experts' input, which is the output of an
-    identity expert (idx[t, k] >= E; without h such pairs add nothing)."""
+    identity expert (idx[t, k] >= E; without h such pairs add nothing).  With ``join`` the result goes into the
+    residual instead of ``out`` (which may be None)."""
     _need(act, "experts act", shape=(None, None, None))
     n, top, F = act.shape
     _need(down, "experts down", act.dtype, (None, None, F))
@@ -1271,14 +1326,15 @@ def moe_down(act: torch.Tensor, down: torch.Tensor, idx: torch.Tensor, weights: 
         raise KernelError(f"experts input: {h.dtype} {tuple(h.shape)}, expected {act.dtype} {(n, H)}")
     _need(idx, "chosen experts", torch.int32, (n, top))
     _need(weights, "expert weights", torch.float32, (n, top))
-    _need(out, "experts out", torch.float32, (n, H))
+    if out is not None or join is None:
+        _need(out, "experts out", torch.float32, (n, H))
     sp, sstr = _parts_of(shared, n, H, "shared expert") if shared is not None else (0, 0)
     if shared_gate is not None:
         _need(shared_gate, "shared gate", torch.float32, (n,))
     _check(_fn("moe", "cpmcu_moe_down")(_p(act), c_int(_code(act)), _p(down), _p(idx), _p(weights), _p(shared),
                                         c_int(_code(shared) if shared is not None else 0), c_int(sp), c_long(sstr),
                                         _p(shared_gate), _p(h), c_long(ldh), c_int(E), _p(out), c_int(n), c_int(H),
-                                       c_int(F), c_int(top), _stream()))
+                                       c_int(F), c_int(top), *_join_args(join, n, H, act.dtype), _stream()))
 
 
 MOE_TILE = 64
@@ -1296,9 +1352,9 @@ def moe_experts_mfma_ok(h: torch.Tensor, expert_size: int, n_tiles: int) -> bool
 
 
 def moe_experts_mfma(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, idx: torch.Tensor, weights: torch.Tensor,
-                     out: torch.Tensor, act: torch.Tensor, y: torch.Tensor, rows: torch.Tensor, tile_expert: torch.Tensor,
+                     out: Optional[torch.Tensor], act: torch.Tensor, y: torch.Tensor, rows: torch.Tensor, tile_expert: torch.Tensor,
                      n_tiles: torch.Tensor, shared: Optional[torch.Tensor] = None,
-                     shared_gate: Optional[torch.Tensor] = None, activation="silu"):
+                     shared_gate: Optional[torch.Tensor] = None, activation="silu", join: Optional[Join] = None):
     """moe_gated + moe_down for steps of many tokens, bf16 on the matrix cores: the (token, expert) pairs are grouped
     by expert into tiles of MOE_TILE rows (pairs of identity experts, idx >= E, have none: they add h).  Scratch: act bf16 [n, top, F], y bf16 [n, top, H], rows int32
     [tiles * MOE_TILE], tile_expert int32 [tiles], n_tiles int32 [1], tiles >= moe_tiles(n, top, E)."""
@@ -1310,7 +1366,8 @@ def moe_experts_mfma(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
     _need(idx, "chosen experts", torch.int32, (n, None))
     top = idx.shape[1]
     _need(weights, "expert weights", torch.float32, (n, top))
-    _need(out, "experts out", torch.float32, (n, H))
+    if out is not None or join is None:
+        _need(out, "experts out", torch.float32, (n, H))
     _need(act, "experts act", torch.bfloat16, (n, top, F))
     _need(y, "experts pair outputs", torch.bfloat16, (n, top, H))
     _need(tile_expert, "experts tile map", torch.int32, (None,))
@@ -1326,7 +1383,7 @@ def moe_experts_mfma(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
         _p(h), c_long(ldh), _p(gate_up), _p(down), _p(idx), _p(weights), _p(shared),
         c_int(_code(shared) if shared is not None else 0), c_int(sp), c_long(sstr), _p(shared_gate), _p(act), _p(y),
         _p(rows), _p(tile_expert), _p(n_tiles), c_int(tiles), _p(out), c_int(n), c_int(H), c_int(F), c_int(E), c_int(top),
-        *_act(activation), _stream()))
+        *_act(activation), *_join_args(join, n, H, torch.bfloat16), _stream()))
 
 
 def latent_store(q_out: Optional[torch.Tensor], nh: int, dim: int, rot: int, rank: int, eps: float, positions: torch.Tensor,
@@ -1813,7 +1870,9 @@ def attention_general_mfma(q: torch.Tensor, out: torch.Tensor, nh: int, nkv: int
                            part_o: Optional[torch.Tensor] = None, part_ml: Optional[torch.Tensor] = None,
                            tiles: Optional[torch.Tensor] = None, tokens_per_tile: int = 1, window: int = 0,
                            keep_first: int = 0, sink: Optional[torch.Tensor] = None, v_share: int = 1,
-                           gate: Optional[torch.Tensor] = None, softcap: float = 0.0):
+                           gate: Optional[torch.Tensor] = None, softcap: float = 0.0,
+                           v_inv_freq: Optional[torch.Tensor] = None, head_gate: Optional[torch.Tensor] = None,
+                           interleaved: bool = False):
     """attention_general in bf16 on the matrix cores (key size a multiple of 8 up to 1024, value size up to 512).
     With n_splits > 1 every token's visible keys are shared among n_splits workgroups and merged afterwards;
     part_o float32 [n, nh, n_splits, hdv] and part_ml float32 [n, nh, n_splits, 2] are its scratch.
@@ -1821,7 +1880,8 @@ def attention_general_mfma(q: torch.Tensor, out: torch.Tensor, nh: int, nkv: int
     kv head): runs of at most tokens_per_tile consecutive tokens of one sequence,
     which share a matrix-core tile (tokens_per_tile * heads a kv head <= 16).  out is bfloat16, or float32 for a
     consumer that goes on in float (a difference of two maps).  gate (bfloat16 [n, nh*hdv], may be a column slice
-    of a wider projection): the output is multiplied element by element with sigmoid(gate) before it is written."""
+    of a wider projection): the output is multiplied element by element with sigmoid(gate) before it is written.
+    v_inv_freq / head_gate / interleaved, with n_splits > 1 only: the merge of the shares does head_output's work."""
     _need(q, "attention q", torch.bfloat16, (None, nh * hdk))
     n = q.shape[0]
     if out.dtype not in (torch.bfloat16, torch.float32):
@@ -1847,6 +1907,13 @@ def attention_general_mfma(q: torch.Tensor, out: torch.Tensor, nh: int, nkv: int
         ld_gate = _ld(gate, "attention gate")
         if gate.dtype != torch.bfloat16 or tuple(gate.shape) != (n, nh * hdv):
             raise KernelError(f"attention gate: {gate.dtype} {tuple(gate.shape)}, expected bfloat16 {(n, nh * hdv)}")
+    ld_head = 0
+    if v_inv_freq is not None:
+        _need(v_inv_freq, "attention value inv_freq", torch.float32, (hdv // 2,))
+    if head_gate is not None:
+        ld_head = _ld(head_gate, "attention head gate")
+        if head_gate.dtype != torch.bfloat16 or tuple(head_gate.shape) != (n, nh):
+            raise KernelError(f"attention head gate: {head_gate.dtype} {tuple(head_gate.shape)}, expected bfloat16 {(n, nh)}")
     _check(_fn("attention_general", "cpmcu_attention_general_mfma")(
         _p(q), _p(out), c_int(1 if out.dtype == torch.float32 else 0), _p(part_o), _p(part_ml), c_int(n), c_int(nh),
         c_int(nkv), c_int(hdk), c_int(hdv),
@@ -1854,7 +1921,8 @@ def attention_general_mfma(q: torch.Tensor, out: torch.Tensor, nh: int, nkv: int
         c_int(keep_first), _p(sink), _p(kpool), _p(vpool),
         _p(page_table), c_int(page_table.shape[1]), c_int(page_size), _p(positions), _p(tok_slot), c_int(n_splits),
         _p(tiles), c_int(tiles.shape[0] if tiles is not None else 0), c_int(tokens_per_tile), c_int(v_share),
-        _p(gate), c_long(ld_gate), c_float(softcap or 0.0), _stream()))
+        _p(gate), c_long(ld_gate), c_float(softcap or 0.0), _p(v_inv_freq), c_int(1 if interleaved else 0), _p(head_gate),
+        c_long(ld_head), _stream()))
 
 
 def attention_general_tokens_per_tile(n_tokens: int, nh: int, nkv: int, pool_hdv: int) -> int:
@@ -1879,14 +1947,24 @@ def reserve_attention_general(ws, dtype, nh: int, nkv: int, hdv: int, pool_hdv: 
         ws.get("attn.gpart_ml", (most, nh, 2), torch.float32)
 
 
+class HeadFinish:
+    """head_output's work as attention_any takes it along: the finished heads (``out``), the frequencies that turn rotated
+    values back, the gate a head (either may be None) and the layout of pairs."""
+    __slots__ = ("out", "inv_freq", "gate", "interleaved")
+
+    def __init__(self, out: torch.Tensor, inv_freq: Optional[torch.Tensor], gate: Optional[torch.Tensor], interleaved: bool):
+        self.out, self.inv_freq, self.gate, self.interleaved = out, inv_freq, gate, bool(interleaved)
+
+
 def attention_any(q, out, nh, nkv, hdk, hdv, scale, kpool, vpool, page_table, page_size, ctx, chunk: int = 0,
                   window: int = 0, keep_first: int = 0, sink: Optional[torch.Tensor] = None, v_share: int = 1,
-                  gate: Optional[torch.Tensor] = None, softcap: float = 0.0) -> bool:
+                  gate: Optional[torch.Tensor] = None, softcap: float = 0.0, finish: Optional["HeadFinish"] = None) -> bool:
     """Attention with key and value sizes of their own and an optional mask (chunks, or a sliding window with kept
     first tokens) and softmax sink, with the kernel that suits the step; writes ``out`` [n, nh*hdv] (q's type, or
     float32).  v_share: runs of that many neighbouring key heads read one value head.  gate [n, nh*hdv]: an output
     gate that the matrix-core kernel applies as it writes (out * sigmoid(gate)); returns whether it did, so that
-    the caller applies it itself after the other kernels.  softcap c > 0: scaled scores pass c tanh(s / c)."""
+    the caller applies it itself after the other kernels.  finish: what head_output does, into a tensor of its own; the
+    merge of split keys does it on its way (out is then not written), and the return value says so.  softcap c > 0: scaled scores pass c tanh(s / c)."""
     pool_hdv = vpool.shape[2] // _value_heads(nkv, v_share)
     if (hdk == hdv and chunk == 0 and window == 0 and sink is None and hdk <= 256 and hdk % 16 == 0
             and kpool.shape[2] == nkv * hdk and v_share == 1 and not softcap and out.dtype == q.dtype):
@@ -1912,10 +1990,12 @@ def attention_any(q, out, nh, nkv, hdk, hdv, scale, kpool, vpool, page_table, pa
                 tiles = ctx.extras.get(key)
                 if tiles is None:
                     tiles = ctx.extras[key] = prefill_tiles(ctx.q_lens, tpt, q.device)
-        attention_general_mfma(q, out, nh, nkv, hdk, hdv, scale, kpool, vpool, page_table, page_size, ctx.positions,
-                               ctx.tok_slot, chunk, splits, part_o, part_ml, tiles, tpt, window, keep_first, sink, v_share,
-                               gate, softcap)
-        return gate is not None
+        there = finish is not None and splits > 1 and finish.out.dtype == torch.bfloat16
+        kw = dict(v_inv_freq=finish.inv_freq, head_gate=finish.gate, interleaved=finish.interleaved) if there else {}
+        attention_general_mfma(q, finish.out if there else out, nh, nkv, hdk, hdv, scale, kpool, vpool, page_table, page_size,
+                               ctx.positions, ctx.tok_slot, chunk, splits, part_o, part_ml, tiles, tpt, window, keep_first,
+                               sink, v_share, gate, softcap, **kw)
+        return gate is not None or there
     if out.dtype != q.dtype:
         # the plain kernel writes the type it reads: through scratch of that type
         tmp = ctx.ws.get("attn.gout_plain", tuple(out.shape), q.dtype)

@@ -403,21 +403,27 @@ class GeneralAttention(Mixer):
         finish = v_freq is not None or self.head_gate_off is not None
         out = ctx.ws.get("attn.heads" if finish else "attn.out", (n, nh * dv), torch.float32 if finish else self.rt.dtype)
         gate = qkv[:, self.gate_off:self.gate_off + nh * dv] if self.gate_off is not None else None
+        fin = None
+        if finish:
+            head_gate = qkv[:, self.head_gate_off:self.head_gate_off + nh] if self.head_gate_off is not None else None
+            fin = ops.HeadFinish(ctx.ws.get("attn.out", (n, nh * dv), self.rt.dtype), v_freq, head_gate, self.interleaved)
         with ctx.timed("attn_core"):
-            # the matrix-core kernel (and the merge of split keys) applies the gate as it writes
-            gated_there = ops.attention_any(q, out, nh, nkv, dk, dv, self.scale, cache.streams["k"], cache.streams["v"],
-                                            cache.page_table, cache.page_size, ctx, chunk=self.chunk, window=self.window,
-                                            keep_first=self.keep_first, sink=self.sink, gate=gate, softcap=self.softcap)
-        if gate is not None and not gated_there:
+            # the matrix-core kernel (and the merge of split keys) applies the gate as it writes; the merge also turns
+            # rotated values back and applies a gate a head
+            done_there = ops.attention_any(q, out, nh, nkv, dk, dv, self.scale, cache.streams["k"], cache.streams["v"],
+                                           cache.page_table, cache.page_size, ctx, chunk=self.chunk, window=self.window,
+                                           keep_first=self.keep_first, sink=self.sink, gate=gate, softcap=self.softcap,
+                                           finish=fin)
+        if gate is not None and not done_there:
             with ctx.timed("attn_gate"):
                 gated = ctx.ws.get("attn.gated", (n, nh * dv), self.rt.dtype)
                 ops.sigmoid_gate(out, gate, gated)
                 out = gated
-        if finish:
-            with ctx.timed("attn_gate"):
-                heads, out = out, ctx.ws.get("attn.out", (n, nh * dv), self.rt.dtype)
-                head_gate = qkv[:, self.head_gate_off:self.head_gate_off + nh] if self.head_gate_off is not None else None
-                ops.head_output(heads, out, nh, dv, ctx.positions, v_freq, head_gate, interleaved=self.interleaved)
+        if fin is not None:
+            if not done_there:
+                with ctx.timed("attn_gate"):
+                    ops.head_output(out, fin.out, nh, dv, ctx.positions, fin.inv_freq, fin.gate, interleaved=fin.interleaved)
+            out = fin.out
         with ctx.timed("attn_o"):
             branch = self.o.forward(out, ctx, "attn.o", out_dtype=torch.float32, partials=True)
         return BiasedBranch(branch, self.o.bias, ctx, "attn.o") if self.o.bias is not None else branch

@@ -408,6 +408,13 @@ class FeedForward(Part):
 
     # True if forward accepts ``defer_last=True`` and may then return a DeferredBranch
     can_defer_last = False
+    # True (set in the class that defines ``forward``) if forward accepts ``join=`` (ops.Join): its result, the other
+    # result of a parallel layer and the residual are then summed in its last kernel, and it returns None.  ``joins``
+    # says whether it would for a given other result
+    can_join = False
+
+    def joins(self, other: Optional[torch.Tensor]) -> bool:
+        return self.can_join
 
 
 def forward_declares(part: Part, flag: str) -> bool:

@@ -231,6 +231,7 @@ class ParallelBlock(Block):
             raise ValueError("parallel: one input convolution for every sub-layer")
         self.norm, self.mixer, self.feed_forward, self.hidden_size = norm, mixer, feed_forward, hidden_size
         self.input_conv, self.token_input = input_conv, token_input
+        self._ff_joins = feed_forward is not None and forward_declares(feed_forward, "can_join")
 
     def parts(self) -> List[Part]:
         return [p for p in (self.norm, self.input_conv, self.mixer, self.feed_forward, self.token_input) if p is not None]
@@ -255,19 +256,25 @@ class ParallelBlock(Block):
                                         tag="block.h")]
         with ctx.timed("attn"):
             a, a_bias = _with_bias(self.mixer.forward(hs[0], ctx, cache, writes_cache))
+        x = stream.x
+        copy = None if self.token_input is None else ctx.ws.get("block.x", tuple(x.shape), self.rt.dtype)
         f = f_bias = None
-        if self.feed_forward is not None:
+        joined = self._ff_joins and self.feed_forward.joins(a)
+        if joined:                        # the feed-forward's last kernel ends the layer's sum in the residual
+            with ctx.timed("ffn"):
+                self.feed_forward.forward(hs[-1], ctx, join=ops.Join(x, a, a_bias, copy))
+        elif self.feed_forward is not None:
             with ctx.timed("ffn"):
                 f, f_bias = _with_bias(self.feed_forward.forward(hs[-1], ctx))
-        x = stream.x
-        with ctx.timed("residual"):
-            if self.token_input is None:
-                out = ctx.ws.get("block.sum", tuple(x.shape), torch.float32)
-                ops.scaled_branches(a, a_bias, None, 1.0, f, f_bias, None, 1.0, out)
-            else:
-                out = ctx.ws.get("block.x", tuple(x.shape), self.rt.dtype)
-                ops.add_rows(x, a, a_bias, f, f_bias, out)
-        stream.pending = out if self.token_input is None else self.token_input.forward(out, ctx)
+        pending = None
+        if not joined:
+            with ctx.timed("residual"):
+                if self.token_input is None:
+                    pending = ctx.ws.get("block.sum", tuple(x.shape), torch.float32)
+                    ops.scaled_branches(a, a_bias, None, 1.0, f, f_bias, None, 1.0, pending)
+                else:
+                    ops.add_rows(x, a, a_bias, f, f_bias, copy)
+        stream.pending = pending if self.token_input is None else self.token_input.forward(copy, ctx)
         stream.pending_scale = 1.0
 
 

@@ -163,24 +163,39 @@ class RoutedExpertsFFN(FeedForward):
         self.router = f32(self.names["router"])
         self.correction = f32(self.names["correction"]) if self.names.get("correction") else None
         self.shared_scale = f32(self.names["shared_scale"]).reshape(-1) if self.shared_gated else None
+        # steps of many tokens: the router as a product of the library's, bf16 operands summed in float.  A bf16 weight
+        # times a bf16 row is exact in float, so this is the float product of the kernel for few tokens
+        self.router_rows = None
+        named = [tensors[self.names[k]] for k in ("router", "shared_scale") if self.names.get(k) and (k == "router" or self.shared_gated)]
+        if rt.dtype == torch.bfloat16 and all(t.dtype == torch.bfloat16 for t in named):
+            last = named[1].reshape(1, -1) if self.shared_gated else torch.zeros_like(named[0][:1])
+            self.router_rows = torch.cat([named[0], last]).contiguous()       # [routes + 1, H], as the logits lie
         # an expert's gate rows, then its up rows: [E, 2F, H]; down: [E, H, F]
         self.gate_up = torch.stack([torch.cat([tensors[self._expert(e, "gate")], tensors[self._expert(e, "up")]], 0)
                                     for e in range(self.experts)]).to(rt.dtype).contiguous()
         self.down = torch.stack([tensors[self._expert(e, "down")] for e in range(self.experts)]).to(rt.dtype).contiguous()
 
-    def forward(self, h: torch.Tensor, ctx: StepContext):
+    can_join = True
+
+    def joins(self, other) -> bool:
+        return other is None or other.dim() == 2 or other.shape[0] <= ops.JOIN_MAX_PARTS
+
+    def forward(self, h: torch.Tensor, ctx: StepContext, join=None):
         n = h.shape[0]
         idx = ctx.ws.get("moe.idx", (n, self.top), torch.int32)
         wts = ctx.ws.get("moe.weights", (n, self.top), torch.float32)
         sg = ctx.ws.get("moe.shared_gate", (n,), torch.float32) if self.shared_gated else None
         logits = ctx.ws.get("moe.logits", (n, self.routes + 1), torch.float32)
         with ctx.timed("moe_route"):
+            many = self.router_rows is not None and n > ops.SKINNY_MAX_ROWS
+            if many:
+                torch.mm(h, self.router_rows.t(), out_dtype=torch.float32, out=logits)
             ops.moe_route(h, self.router, self.correction, self.shared_scale, self.groups[0], self.groups[1], self.top,
                           idx, wts, sg, logits, score=self.score, group_score=self.group_score,
-                          weight_scale=self.weight_scale, normalize=self.normalize)
+                          weight_scale=self.weight_scale, normalize=self.normalize, logits_ready=many)
         shared = self.shared.forward(h, ctx) if self.shared is not None else None
         act = ctx.ws.get("moe.act", (n, self.top, self.expert_size), self.rt.dtype)
-        out = ctx.ws.get("moe.out", (n, self.hidden_size), torch.float32)
+        out = ctx.ws.get("moe.out", (n, self.hidden_size), torch.float32) if join is None else None
         tiles = ops.moe_tiles(n, self.top, self.experts)
         with ctx.timed("moe_experts"):
             # few tokens read an expert's matrices once for every token that chose it; from about one and a half
@@ -193,9 +208,9 @@ class RoutedExpertsFFN(FeedForward):
                 tile_expert = ctx.ws.get("moe.tile_expert", (tiles,), torch.int32)
                 n_tiles = ctx.ws.get("moe.n_tiles", (1,), torch.int32)
                 ops.moe_experts_mfma(h, self.gate_up, self.down, idx, wts, out, act, y, rows, tile_expert, n_tiles,
-                                     shared, sg, activation=self.activation)
+                                     shared, sg, activation=self.activation, join=join)
             else:
                 # few tokens: an expert's weights stream once for every token that chose it
                 ops.moe_gated(h, self.gate_up, idx, act, activation=self.activation)
-                ops.moe_down(act, self.down, idx, wts, out, shared, sg, h=h)
+                ops.moe_down(act, self.down, idx, wts, out, shared, sg, h=h, join=join)
         return out

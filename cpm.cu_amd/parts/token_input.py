@@ -52,9 +52,12 @@ class TokenInput(Part):
         """x [n, H]: the residual in the engine's element type."""
         n = x.shape[0]
         with ctx.timed("token_input"):
-            z = self.gate.forward(x, ctx, "side.gate", out_dtype=torch.float32 if n <= ops.SKINNY_MAX_ROWS else None,
-                                  partials=True)
             g = ctx.ws.get("side.act", (n, self.dim), self.rt.dtype)
-            ops.gated_lookup(z, self.source.table, self.offset, ctx.token_ids, g, self.activation)
+            if n <= ops.LOOKUP_STRIP_ROWS and self.gate.tiled is not None and x.shape[1] % 8 == 0:
+                ops.lookup_strip(x, self.gate.tiled, self.source.table, self.offset, ctx.token_ids, g, self.activation)
+            else:
+                z = self.gate.forward(x, ctx, "side.gate", out_dtype=torch.float32 if n <= ops.SKINNY_MAX_ROWS else None,
+                                      partials=True)
+                ops.gated_lookup(z, self.source.table, self.offset, ctx.token_ids, g, self.activation)
             y = self.proj.forward(g, ctx, "side.proj", out_dtype=torch.float32, partials=True)
         return NormedBranch(y, self.norm, ctx, "side.norm")

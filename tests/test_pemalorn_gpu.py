@@ -239,8 +239,9 @@ def test_residual_stream_after_every_layer_run(models, name):
     def spy(i):
         def f(stream, ctx, cache, writes_cache=True):
             originals[i](stream, ctx, cache, writes_cache)
-            y = branch_tensor(stream.take_pending()).double()
-            seen.append((stream.x.double() + (y.sum(0) if y.dim() == 3 else y)).cpu())
+            y = branch_tensor(stream.take_pending())          # None: the layer's last kernel ended the sum itself
+            y = torch.zeros_like(stream.x) if y is None else y
+            seen.append((stream.x.double() + (y.double().sum(0) if y.dim() == 3 else y.double())).cpu())
         return f
     try:
         for i, b in enumerate(blocks):

@@ -203,6 +203,20 @@ def test_gated_lookup_of_the_token_table(dtype, D, off, parts):
     close(out, plain.gelu_tanh(zz) * table.double()[ids][:, off:off + D], dtype)
 
 
+@pytest.mark.parametrize("n, K, D, off", [(1, 96, 12, 24), (8, 4096, 256, 256), (16, 1000, 40, 3), (5, 64, 1, 0), (3, 200, 17, 5)])
+def test_product_and_lookup_in_one_launch(n, K, D, off):
+    from cpmcu_amd import ops
+    g = torch.Generator().manual_seed(81)
+    x, w = torch.randn(n, K, generator=g).bfloat16(), (torch.randn(D, K, generator=g) * K ** -0.5).bfloat16()
+    table, ids = torch.randn(23, off + D + 2, generator=g).bfloat16(), torch.randint(0, 23, (n,), generator=g)
+    out = torch.empty(n, D, dtype=torch.bfloat16, device=DEV)
+    ops.lookup_strip(dev(x), ops.TiledWeight(dev(w)), dev(table), off, i32(ids.tolist()), out)
+    close(out, plain.gelu_tanh(x.double() @ w.double().T) * table.double()[ids][:, off:off + D], "bfloat16")
+    with pytest.raises(ops.KernelError, match="tokens"):
+        ops.lookup_strip(torch.zeros(17, K, dtype=torch.bfloat16, device=DEV), ops.TiledWeight(dev(w)), dev(table), off,
+                         torch.zeros(17, dtype=torch.int32, device=DEV), torch.empty(17, D, dtype=torch.bfloat16, device=DEV))
+
+
 # ---------------------------------------------------------------------------
 # rotated values, a number a head on the scores, a sink and a gate a head
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
@@ -275,6 +289,15 @@ def test_rotated_values_through_the_cache(dtype, shape):
         ops.attention_general_mfma(q_out[a:b], heads, H, G, d, dv, scale, kp, vp, dev(table), page, pos[a:b], slot[a:b], 0, splits,
                                    po, pm, tiles, tpt, sink=dev(sink))
         close(finish(a, b, heads), want[a:b], "bfloat16", scale=float(want.abs().max()), what=f"matrix cores rows {a}..{b} splits {splits} tiled {tiled}")
+        if splits > 1:               # the merge of the shares turns back and gates on its way
+            out = torch.empty(b - a, H * dv, dtype=torch.bfloat16, device=DEV)
+            ops.attention_general_mfma(q_out[a:b], out, H, G, d, dv, scale, kp, vp, dev(table), page, pos[a:b], slot[a:b], 0, splits,
+                                       po, pm, sink=dev(sink), v_inv_freq=freq(dv), head_gate=gcol[a:b])
+            close(out, want[a:b], "bfloat16", scale=float(want.abs().max()), what=f"merge rows {a}..{b} splits {splits}")
+            ops.attention_general_mfma(q_out[a:b], out, H, G, d, dv, scale, kp, vp, dev(table), page, pos[a:b], slot[a:b], 0, splits,
+                                       po, pm, sink=dev(sink), head_gate=gcol[a:b])
+            gated = heads.double().cpu().reshape(b - a, H, dv) * torch.sigmoid(gate[a:b].double())[:, :, None]
+            close(out, gated.reshape(b - a, H * dv), "bfloat16", what="merge with the gate alone")
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
@@ -447,6 +470,27 @@ def test_experts_and_identity_experts(dtype, n, H, F, E, I, top):
     ops.moe_gated(hd, gu, idx, act)
     ops.moe_down(act, dn, idx, wts, out, h=hd)
     close(out, want, dtype, what="few tokens")
+    # the router's products by the library, the choice from them
+    if dtype == "bfloat16":
+        rows = torch.cat([W["router"], torch.zeros(1, H, dtype=torch.bfloat16)])
+        logits = torch.empty(n, E + I + 1, device=DEV)
+        torch.mm(hd, dev(rows).t(), out_dtype=torch.float32, out=logits)
+        idx3, wts3 = torch.empty_like(idx), torch.empty_like(wts)
+        ops.moe_route(hd, dev(W["router"].float()), dev(W["correction"].float()), None, 1, 1, top, idx3, wts3, None, logits,
+                      normalize=False, logits_ready=True)
+        assert torch.equal(idx3.cpu().long()[sure], idx_want[sure])
+        close(wts3[dev(sure)], w_want[sure], "float32", scale=1.0)
+
+    def joined(run):
+        """The same with the layer's sum ended there: another result (float parts, a bf16 tensor with a bias, none)."""
+        for a, bias in ((torch.randn(5, n, H, generator=g), None), (torch.randn(n, H, generator=g).bfloat16(), torch.randn(H, generator=g)), (None, None)):
+            x0 = torch.randn(n, H, generator=g)
+            x, copy = dev(x0.clone()), torch.empty(n, H, dtype=DT[dtype], device=DEV)
+            run(ops.Join(x, dev(a) if a is not None else None, dev(bias) if bias is not None else None, copy))
+            total = x0.double() + want + (0 if a is None else (a.double().sum(0) if a.dim() == 3 else a.double())) + (0 if bias is None else bias.double())
+            close(x, total, dtype, scale=float(want.abs().max()) if dtype == "bfloat16" else None, what="joined")
+            close(copy, total, dtype, what="copy of the joined residual")
+    joined(lambda j: ops.moe_down(act, dn, idx, wts, None, h=hd, join=j))
     tiles = ops.moe_tiles(n, top, E)
     if ops.moe_experts_mfma_ok(hd, F, tiles):
         out2 = torch.empty(n, H, device=DEV)
@@ -455,6 +499,8 @@ def test_experts_and_identity_experts(dtype, n, H, F, E, I, top):
         ops.moe_experts_mfma(hd, gu, dn, idx, wts, out2, act2, y, torch.empty(tiles * ops.MOE_TILE, dtype=torch.int32, device=DEV),
                              torch.empty(tiles, dtype=torch.int32, device=DEV), torch.empty(1, dtype=torch.int32, device=DEV))
         close(out2, want, dtype, what="grouped")
+        joined(lambda j: ops.moe_experts_mfma(hd, gu, dn, idx, wts, None, act2, y, torch.empty(tiles * ops.MOE_TILE, dtype=torch.int32, device=DEV),
+                                              torch.empty(tiles, dtype=torch.int32, device=DEV), torch.empty(1, dtype=torch.int32, device=DEV), join=j))
 
 
 def test_refusals():
