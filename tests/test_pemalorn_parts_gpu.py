@@ -412,7 +412,7 @@ def test_product_over_heads_with_a_gate_a_feature(dtype, M, H, N, K):
         close(out, want, dtype)
 
 
-@pytest.mark.parametrize("dims, base, scaling", [(8, 500.0, (4.0, 64, 16.0, 1.0)), (16, 1e6, (2.0, 1024, 32.0, 1.0)), (2, 20.0, (8.0, 32, 4.0, 1.0)),
+@pytest.mark.parametrize("dims, base, scaling", [(8, 500.0, (4.0, 64, 16.0, 1.0)), (24, 2e5, (3.0, 700, 20.0, 1.5)), (2, 20.0, (8.0, 32, 4.0, 1.0)),
                                                  (64, 10000.0, (40.0, 4096, 32.0, 1.0))])
 def test_stretched_frequencies(dims, base, scaling):
     from cpmcu_amd.parts import POSITION_ENCODINGS, Runtime, Workspace

@@ -32,7 +32,7 @@ def tiny_s():
              "mlp": {"kind": "moe", "expert": {"ff": 16}, "router": {"experts": 3, "identity": 5, "top": 4}}},
             {"type": "latent_attention", "mixer": {
                 "heads": 2, "dim": 32, "rot_dim": 8, "vdim": 32, "q_rank": 24, "kv_rank": 64, "scale": 0.18,
-                "rot": {"base": 1000.0, "dims": 8, "scaling": {"factor": 2.0, "original": 1024, "fast": 32.0, "slow": 1.0}}},
+                "rot": {"base": 1000.0, "dims": 8, "scaling": {"factor": 3.0, "original": 500, "fast": 20.0, "slow": 0.7}}},
              "mlp": {"kind": "moe", "expert": {"ff": 32}, "router": {"experts": 8, "identity": 2, "top": 1}}},
         ],
     }
