@@ -5,3 +5,4 @@ from .gumodra import GumodraConfig
 from .sagedra import SagedraConfig
 from .nelutar import NelutarConfig
 from .pemalorn import PemalornConfig
+from .tirizen import TirizenConfig

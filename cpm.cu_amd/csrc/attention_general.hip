@@ -703,7 +703,8 @@ extern "C" const char* cpmcu_qkv_rotate_store(const void* qkv, long ld, int dtyp
 //   * with norm_after q and k heads are rotated first and then divided by their root mean square (times the
 //     weight, if one is given);
 //   * with interleaved the rotation pairs neighbouring features (2i, 2i + 1) instead of (i, i + rot_dims/2);
-//   * q_scale (a number a query head) multiplies the finished query head, before it is rounded;
+//   * q_scale (a number a query head) multiplies the finished query head, before it is rounded, and so does the
+//     position's temperature 1 + temp_coef ln(floor((p + 1) / temp_every) + 1) (temp_every 0: none);
 //   * v_inv_freq (dv/2 frequencies): value heads of their own are rotated as well, over all dv features, in the same
 //     layout of pairs and without a magnitude (head_output_kernel turns what the attention makes of them back).
 // The projection's rows may be float where the cache is bfloat16 (rows that a convolution wrote).
@@ -714,7 +715,7 @@ __global__ __launch_bounds__(64) void qkv_norm_rotate_store_kernel(
     int values_from_keys, const int* __restrict__ positions, const int* __restrict__ tok_slot,
     const float* __restrict__ inv_freq, float mag, T* __restrict__ kpool, T* __restrict__ vpool, PagedView pv,
     int pool_hdk, int pool_hdv, int norm_after, int interleaved, const float* __restrict__ q_scale,
-    const float* __restrict__ v_inv_freq) {
+    const float* __restrict__ v_inv_freq, float temp_coef, int temp_every) {
     __shared__ float hs[AG_MAX_HD];
     const long t = blockIdx.x;
     const int y = blockIdx.y, lane = threadIdx.x;
@@ -769,8 +770,9 @@ __global__ __launch_bounds__(64) void qkv_norm_rotate_store_kernel(
         const float r = 1.0f / sqrtf(wave_sum(ss) / (float)width + eps);
         for (int i = lane; i < width; i += 64) hs[i] = hs[i] * r * nw[i];
     }
-    if (is_q && q_scale) {
-        const float qs = q_scale[h];
+    if (is_q && (q_scale || temp_every > 0)) {
+        const float qs = (q_scale ? q_scale[h] : 1.0f) *
+                         (temp_every > 0 ? 1.0f + temp_coef * logf((float)((pos + 1) / temp_every) + 1.0f) : 1.0f);
         for (int i = lane; i < width; i += 64) hs[i] *= qs;
     }
     __syncthreads();
@@ -786,8 +788,10 @@ extern "C" const char* cpmcu_qkv_norm_rotate_store(const void* qkv, long ld, int
                                                    const float* inv_freq, float mag, void* kpool, void* vpool,
                                                    const int* page_table, int table_width, int page_size, int pool_hdk,
                                                    int pool_hdv, int write_kv, int norm_after, int interleaved, int in_dtype,
-                                                   const float* q_scale, const float* v_inv_freq, hipStream_t stream) {
+                                                   const float* q_scale, const float* v_inv_freq, float temp_coef,
+                                                   int temp_every, hipStream_t stream) {
     CPMCU_REQUIRE(n > 0 && nh > 0 && nkv > 0 && dk > 0 && dv > 0, "qkv_norm_rotate_store: empty shape");
+    CPMCU_REQUIRE(temp_every >= 0, "qkv_norm_rotate_store: a temperature step of %d positions", temp_every);
     CPMCU_REQUIRE(!v_inv_freq || (dv % 2 == 0 && !values_from_keys), "qkv_norm_rotate_store: rotated values have heads of their own of an even size (%d)", dv);
     CPMCU_REQUIRE(dk <= AG_MAX_HD && dv <= AG_MAX_HD, "qkv_norm_rotate_store: key size %d / value size %d (up to %d are taken)",
                   dk, dv, AG_MAX_HD);
@@ -807,7 +811,7 @@ extern "C" const char* cpmcu_qkv_norm_rotate_store(const void* qkv, long ld, int
     qkv_norm_rotate_store_kernel<ITv, Tv><<<grid, 64, 0, stream>>>(                                                  \
         (const ITv*)qkv, ld, bias, (Tv*)q_out, nh, nkv, dk, dv, rot_dims, q_norm_w, k_norm_w, eps, values_from_keys, \
         positions, tok_slot, inv_freq, mag, (Tv*)kpool, (Tv*)vpool, pv, pool_hdk, pool_hdv, norm_after, interleaved, \
-        q_scale, v_inv_freq)
+        q_scale, v_inv_freq, temp_coef, temp_every)
     // dtype: the cache's and q_out's element type; in_dtype: the projection rows' (float rows may feed a bfloat16 cache)
     if (dtype == CPMCU_F32 && in_dtype == CPMCU_F32) LAUNCH(float, float);
     else if (dtype == CPMCU_BF16 && in_dtype == CPMCU_BF16) LAUNCH(bf16_t, bf16_t);
@@ -815,6 +819,122 @@ extern "C" const char* cpmcu_qkv_norm_rotate_store(const void* qkv, long ld, int
     else CPMCU_FAIL("qkv_norm_rotate_store: unsupported dtypes in=%d out=%d", in_dtype, dtype);
 #undef LAUNCH
     CPMCU_LAUNCH_CHECK("qkv_norm_rotate_store");
+    return nullptr;
+}
+
+// The same for designs that norm the whole projection of the queries, and of the keys, before it is split into heads:
+// grid (tokens, 3) (1 without the cache), a workgroup for a token's queries, one for its keys, one for its values.
+// The rows may come as `nparts` float partial sums of a split product (part_stride apart); a row waits in LDS as float
+// between its two passes (the sum of squares, then norm and copy), a wavefront a head in the second.
+//   * q row: / sqrt(mean(q^2) + eps) * q_norm_w (nh*dk numbers) * (1 + temp_coef ln(floor((p + 1) / temp_every) + 1))
+//     (temp_every 0: no temperature), then a rotation of each head's first rot_dims features; k row the same with
+//     k_norm_w (nkv*dk numbers) and no temperature, into the key pages; v copied into the value pages.
+//   * gate_out (may be absent): the nh numbers behind the row's last v (behind q without the cache), copied.
+template <typename IT, typename T>
+__global__ __launch_bounds__(1024) void qkv_row_norm_store_kernel(
+    const IT* __restrict__ qkv, long ld, int nparts, long part_stride, T* __restrict__ q_out, int nh, int nkv, int dk, int dv,
+    int rot_dims, const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w, float eps, float temp_coef,
+    int temp_every, const int* __restrict__ positions, const int* __restrict__ tok_slot, const float* __restrict__ inv_freq,
+    float mag, T* __restrict__ kpool, T* __restrict__ vpool, PagedView pv, int pool_hdk, int pool_hdv, int interleaved,
+    long gate_col, T* __restrict__ gate_out) {
+    extern __shared__ float row_s[];
+    __shared__ float red[17];
+    const long t = blockIdx.x;
+    const int what = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+    const int pos = positions[t];
+    const int heads = what == 0 ? nh : nkv, hd = what == 2 ? dv : dk;
+    const int width = heads * hd;
+    const IT* src = qkv + t * ld + (what == 0 ? 0 : (long)nh * dk + (what == 2 ? (long)nkv * dk : 0));
+    auto at = [&](const IT* p) {
+        float v = to_f32(p[0]);
+        for (int s = 1; s < nparts; ++s) v += to_f32(p[s * part_stride]);
+        return v;
+    };
+    float ss = 0.f;
+    if (nparts <= 1) {
+        for (int i = threadIdx.x; i < width; i += blockDim.x) {
+            const float v = to_f32(src[i]);
+            row_s[i] = v;
+            ss += v * v;
+        }
+    } else {
+        for (int i = threadIdx.x; i < width; i += blockDim.x) {
+            float v = 0.f;                          // eight parts' loads in flight
+            for (int f = 0; f < nparts; f += 8) {
+                float u[8];
+#pragma unroll
+                for (int j = 0; j < 8; ++j) u[j] = to_f32(src[(long)min(f + j, nparts - 1) * part_stride + i]);
+#pragma unroll
+                for (int j = 0; j < 8; ++j)
+                    if (f + j < nparts) v += u[j];
+            }
+            row_s[i] = v;
+            ss += v * v;
+        }
+    }
+    if (what == 0 && gate_out)
+        for (int i = threadIdx.x; i < nh; i += blockDim.x) gate_out[t * nh + i] = from_f32<T>(at(qkv + t * ld + gate_col + i));
+    if (what == 2) {
+        const long prow = paged_row(pv, tok_slot[t], pos);
+        __syncthreads();
+        for (int h = wave; h < heads; h += nw)
+            rotate_run(row_s + (long)h * dv, vpool + value_index(prow, h, nkv, pool_hdv), dv, 0, pos, inv_freq, 1.0f, DST_VALUES, 0,
+                       lane, 64);
+        return;
+    }
+    float r = 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps);
+    if (what == 0 && temp_every > 0) r *= 1.0f + temp_coef * logf((float)((pos + 1) / temp_every) + 1.0f);
+    const float* nw_ = what == 0 ? q_norm_w : k_norm_w;
+    // (each thread finishes the values it wrote itself)
+    for (int i = threadIdx.x; i < width; i += blockDim.x) row_s[i] *= r * nw_[i];
+    __syncthreads();
+    const long prow = what == 1 ? paged_row(pv, tok_slot[t], pos) : 0;
+    for (int h = wave; h < heads; h += nw) {
+        const float* s = row_s + (long)h * dk;
+        if (what == 0) rotate_run(s, q_out + (t * nh + h) * dk, dk, rot_dims, pos, inv_freq, mag, DST_ROWS, 0, lane, 64, interleaved);
+        else rotate_run(s, kpool + key_index(prow, h, nkv, pool_hdk), dk, rot_dims, pos, inv_freq, mag, DST_KEYS, 0, lane, 64,
+                        interleaved);
+    }
+}
+
+extern "C" const char* cpmcu_qkv_row_norm_store(const void* qkv, int in_dtype, long ld, int nparts, long part_stride, void* q_out,
+                                                int dtype, int n, int nh, int nkv, int dk, int dv, int rot_dims,
+                                                const float* q_norm_w, const float* k_norm_w, float eps, float temp_coef,
+                                                int temp_every, const int* positions, const int* tok_slot,
+                                                const float* inv_freq, float mag, void* kpool, void* vpool,
+                                                const int* page_table, int table_width, int page_size, int pool_hdk,
+                                                int pool_hdv, int write_kv, int interleaved, long gate_col, void* gate_out,
+                                                hipStream_t stream) {
+    CPMCU_REQUIRE(n > 0 && nh > 0 && nkv > 0 && dk > 0 && dv > 0 && nparts > 0, "qkv_row_norm_store: empty shape");
+    CPMCU_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dk && (rot_dims == 0 || inv_freq),
+                  "qkv_row_norm_store: %d rotated features of %d", rot_dims, dk);
+    CPMCU_REQUIRE(temp_every >= 0, "qkv_row_norm_store: a temperature step of %d positions", temp_every);
+    const long row = (long)nh * dk + (write_kv ? (long)nkv * (dk + dv) : 0);
+    CPMCU_REQUIRE(ld >= row && (!gate_out || (gate_col >= row && ld >= gate_col + nh)), "qkv_row_norm_store: rows of %ld too short", ld);
+    CPMCU_REQUIRE(q_norm_w && q_out && positions && (!write_kv || (k_norm_w && tok_slot)), "qkv_row_norm_store: null pointer");
+    CPMCU_REQUIRE(!write_kv || (kpool && vpool && page_table && page_size % 32 == 0 && pool_hdk % 16 == 0 &&
+                                pool_hdv % 16 == 0 && pool_hdk >= dk && pool_hdv >= dv),
+                  "qkv_row_norm_store: the cache takes pages of a multiple of 32 tokens and head sizes in steps of 16");
+    long width = (long)nh * dk;
+    if (write_kv && (long)nkv * dk > width) width = (long)nkv * dk;
+    if (write_kv && (long)nkv * dv > width) width = (long)nkv * dv;
+    CPMCU_REQUIRE(width * 4 <= 60 * 1024, "qkv_row_norm_store: a row of %ld features does not fit the kernel's LDS (up to 15360)", width);
+    PagedView pv{page_table, table_width, page_size};
+    // few tokens: a row over many threads
+    int block = 256;
+    while (n < 256 && block < 1024 && block * 2 <= width) block *= 2;
+    const dim3 grid(n, write_kv ? 3 : 1);
+#define LAUNCH(ITv, Tv)                                                                                                \
+    qkv_row_norm_store_kernel<ITv, Tv><<<grid, block, width * 4, stream>>>(                                            \
+        (const ITv*)qkv, ld, nparts, part_stride, (Tv*)q_out, nh, nkv, dk, dv, rot_dims, q_norm_w, k_norm_w, eps,      \
+        temp_coef, temp_every, positions, tok_slot, inv_freq, mag, (Tv*)kpool, (Tv*)vpool, pv, pool_hdk, pool_hdv,     \
+        interleaved, gate_col, (Tv*)gate_out)
+    if (dtype == CPMCU_F32 && in_dtype == CPMCU_F32) LAUNCH(float, float);
+    else if (dtype == CPMCU_BF16 && in_dtype == CPMCU_BF16) LAUNCH(bf16_t, bf16_t);
+    else if (dtype == CPMCU_BF16 && in_dtype == CPMCU_F32) LAUNCH(float, bf16_t);
+    else CPMCU_FAIL("qkv_row_norm_store: unsupported dtypes in=%d out=%d", in_dtype, dtype);
+#undef LAUNCH
+    CPMCU_LAUNCH_CHECK("qkv_row_norm_store");
     return nullptr;
 }
 

@@ -34,6 +34,7 @@ MODULES: Dict[str, List[str]] = {
     "ssm": ["ssm.hip"],
     "mlstm": ["mlstm.hip"],
     "delta": ["delta.hip"],
+    "gla": ["gla.hip"],
     "moe": ["moe.hip"],
     "rows": ["rows.hip"],
     "attention_general": ["attention_general.hip", "diff_attention.hip"],

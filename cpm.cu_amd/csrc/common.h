@@ -60,6 +60,14 @@ __device__ inline void gate_prepare(float& g, float& up, int act, float limit) {
     }
 }
 __device__ inline float gate_act(float g, int act) { return g / (1.0f + expf(-gate_arg(g, act))); }
+// Nonlinearity of a feed-forward without a gate, act(up): SiLU, the tanh form of GELU, or the square of relu.
+enum { CPMCU_ACT_RELU_SQUARED = 3 };
+#define CPMCU_PLAIN_ACT_KNOWN(act) ((act) == CPMCU_ACT_SILU || (act) == CPMCU_ACT_GELU_TANH || (act) == CPMCU_ACT_RELU_SQUARED)
+__device__ inline float plain_act(float u, int act) {
+    if (act != CPMCU_ACT_RELU_SQUARED) return gate_act(u, act);
+    const float r = fmaxf(u, 0.f);
+    return r * r;
+}
 
 // Max / sum over the four rows of 16 lanes of a wavefront (lanes that differ in bits 4 and 5 only); every
 // lane gets the result.  gfx950's row swaps exchange rows between two registers inside the vector unit:

@@ -9,28 +9,72 @@
 #include "vec4.h"
 
 // ---------------------------------------------------------------------------
-// embedding:  out[r,:] = float(table[ids[r],:]) * scale
+// embedding:  out[s,r,:] = float(table[ids[r],:]) * scale (+ float(pos_table[positions[r],:])), for every copy s
 // (reference: src/model/embedding.cuh:7-20 gathers, elementwise.cuh:34-41 scales)
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict__ ids, float* __restrict__ out,
-                             int H, float scale) {
+                             int H, float scale, const T* __restrict__ pos_table, const int* __restrict__ positions,
+                             int copies, long copy_stride) {
     const long r = blockIdx.x;
     const T* src = table + (long)ids[r] * H;
+    const T* add = pos_table ? pos_table + (long)positions[r] * H : nullptr;
     float* dst = out + r * H;
-    for (int c = threadIdx.x; c < H; c += blockDim.x) dst[c] = to_f32(src[c]) * scale;
+    for (int c = threadIdx.x; c < H; c += blockDim.x) {
+        const float v = to_f32(src[c]) * scale + (add ? to_f32(add[c]) : 0.f);
+        for (int s = 0; s < copies; ++s) dst[s * copy_stride + c] = v;
+    }
 }
 
 extern "C" const char* cpmcu_embed(const void* table, int dtype, const int* ids, float* out, int n, int H, int V,
-                                   float scale, hipStream_t stream) {
-    CPMCU_REQUIRE(n > 0 && H > 0 && V > 0, "embed: empty shape n=%d H=%d V=%d", n, H, V);
+                                   float scale, const void* pos_table, const int* positions, int copies,
+                                   hipStream_t stream) {
+    CPMCU_REQUIRE(n > 0 && H > 0 && V > 0 && copies > 0, "embed: empty shape n=%d H=%d V=%d copies=%d", n, H, V, copies);
+    CPMCU_REQUIRE(!pos_table || positions, "embed: a table of positions without positions");
     CPMCU_REQUIRE(dtype == CPMCU_F32 || dtype == CPMCU_BF16, "embed: unknown dtype %d", dtype);
     const int block = H >= 1024 ? 256 : 64;
     if (dtype == CPMCU_F32)
-        embed_kernel<float><<<n, block, 0, stream>>>((const float*)table, ids, out, H, scale);
+        embed_kernel<float><<<n, block, 0, stream>>>((const float*)table, ids, out, H, scale, (const float*)pos_table, positions,
+                                                     copies, (long)n * H);
     else
-        embed_kernel<bf16_t><<<n, block, 0, stream>>>((const bf16_t*)table, ids, out, H, scale);
+        embed_kernel<bf16_t><<<n, block, 0, stream>>>((const bf16_t*)table, ids, out, H, scale, (const bf16_t*)pos_table,
+                                                      positions, copies, (long)n * H);
     CPMCU_LAUNCH_CHECK("embed");
+    return nullptr;
+}
+
+// ---------------------------------------------------------------------------
+// z <- act(z) in place, for a feed-forward without a gate (plain_act); 8 elements a thread where they are bf16
+// ---------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void activate_kernel(T* __restrict__ z, long total, int act) {
+    for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < total; i += (long)gridDim.x * 256)
+        z[i] = from_f32<T>(plain_act(to_f32(z[i]), act));
+}
+__global__ __launch_bounds__(256) void activate_bf16x8_kernel(uint4* __restrict__ z, long pieces, int act) {
+    for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < pieces; i += (long)gridDim.x * 256) {
+        const uint4 u = z[i];
+        uint32_t w[4] = {u.x, u.y, u.z, u.w};
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            const float a = plain_act(__uint_as_float(w[k] << 16), act), b = plain_act(__uint_as_float(w[k] & 0xffff0000u), act);
+            w[k] = (uint32_t)f32_to_bf16(a).v | ((uint32_t)f32_to_bf16(b).v << 16);
+        }
+        z[i] = make_uint4(w[0], w[1], w[2], w[3]);
+    }
+}
+
+extern "C" const char* cpmcu_activate(void* z, int dtype, long total, int act, hipStream_t stream) {
+    CPMCU_REQUIRE(total > 0 && z, "activate: empty shape");
+    CPMCU_REQUIRE(CPMCU_PLAIN_ACT_KNOWN(act), "activate: unknown nonlinearity %d", act);
+    CPMCU_REQUIRE(dtype == CPMCU_F32 || dtype == CPMCU_BF16, "activate: unknown dtype %d", dtype);
+    const bool vec = dtype == CPMCU_BF16 && total % 8 == 0 && (uintptr_t)z % 16 == 0;
+    const long work = ((vec ? total / 8 : total) + 255) / 256;
+    const unsigned blocks = (unsigned)(work < 16384 ? work : 16384);
+    if (vec) activate_bf16x8_kernel<<<blocks, 256, 0, stream>>>((uint4*)z, total / 8, act);
+    else if (dtype == CPMCU_BF16) activate_kernel<bf16_t><<<blocks, 256, 0, stream>>>((bf16_t*)z, total, act);
+    else activate_kernel<float><<<blocks, 256, 0, stream>>>((float*)z, total, act);
+    CPMCU_LAUNCH_CHECK("activate");
     return nullptr;
 }
 

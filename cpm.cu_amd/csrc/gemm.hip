@@ -269,6 +269,7 @@ extern "C" const char* cpmcu_gemm_nt_heads_mfma(const void* X, long ldx, long hs
 //   MODE 0: Y (float or bf16) = alpha * product
 //   MODE 1: float partial sums of a K-split, part[blockIdx.y][m][N]
 //   MODE 2: rows come in pairs (gate j, up I+j): Y[m][j] = act(gate) * up  (bf16; act: SiLU or the tanh form of GELU)
+//   MODE 3: Y (bf16) = act(product), a nonlinearity without a gate
 // ===========================================================================
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float floatx4_t __attribute__((ext_vector_type(4)));
@@ -479,13 +480,17 @@ __global__ __launch_bounds__(NW * 64) void gemm_skinny_kernel(const bf16_t* __re
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     const int col = out_base[s] + 4 * g + i;
-                    if (col < N) Yp[(long)tok * ldy + col] = from_f32<OT>(alpha * rs_t * acc[s][t][i]);
+                    if (col < N) {
+                        const float v = alpha * rs_t * acc[s][t][i];
+                        Yp[(long)tok * ldy + col] = from_f32<OT>(MODE == 3 ? plain_act(v, act) : v);
+                    }
                 }
         }
     }
 }
 
-// out_mode: 0 = Y[m,N] in out_dtype; 1 = float partial sums Y[ksplit][m][N]; 2 = gated (N = 2*I rows of W, Y[m,I] bf16)
+// out_mode: 0 = Y[m,N] in out_dtype; 1 = float partial sums Y[ksplit][m][N]; 2 = gated (N = 2*I rows of W, Y[m,I] bf16);
+// 3 = Y[m,N] bf16 with a nonlinearity without a gate
 // row_ss (or null): X is x * w of a norm cut by columns, whose sums of squares [M][ss_slices] these are (a
 // slice for every 64 columns after add_norm_columns, for every 16 after proj_add_norm); the output is multiplied
 // by rsqrt(sum of the row's slices / K + eps) row by row.
@@ -497,7 +502,7 @@ extern "C" const char* cpmcu_gemm_skinny(const void* X, long ldx, const void* W,
                                          int out_dtype, int out_mode, int M, int N, int K, int ksplit, float alpha,
                                          int tiled, const float* row_ss, int ss_slices, float eps, int act,
                                          float act_limit, hipStream_t stream) {
-    CPMCU_REQUIRE(CPMCU_ACT_KNOWN(act), "gemm_skinny: unknown nonlinearity %d", act);
+    CPMCU_REQUIRE(out_mode == 3 ? CPMCU_PLAIN_ACT_KNOWN(act) : CPMCU_ACT_KNOWN(act), "gemm_skinny: unknown nonlinearity %d", act);
     CPMCU_REQUIRE(M > 0 && M <= 64, "gemm_skinny: %d rows (1..64 are taken; more rows belong to the tiled product)", M);
     CPMCU_REQUIRE(N > 0 && K > 0 && K % 8 == 0, "gemm_skinny: K=%d must be a positive multiple of 8 (N=%d)", K, N);
     CPMCU_REQUIRE(ldx % 8 == 0 && ldx >= K && (tiled || (ldw % 8 == 0 && ldw >= K)),
@@ -537,6 +542,7 @@ extern "C" const char* cpmcu_gemm_skinny(const void* X, long ldx, const void* W,
     else if (out_mode == 0 && out_dtype == CPMCU_BF16) BY_MT(0, bf16_t, 1, 4);
     else if (out_mode == 1) BY_MT(1, float, 1, 4);
     else if (out_mode == 2) BY_MT(2, bf16_t, 2, 2);
+    else if (out_mode == 3) BY_MT(3, bf16_t, 1, 4);
     else CPMCU_FAIL("gemm_skinny: unknown output mode %d / dtype %d", out_mode, out_dtype);
 #undef BY_MT
 #undef LAUNCH

@@ -5,13 +5,16 @@
 //    choice scores c = s + correction; the experts form `n_groups` equal groups of neighbours, a group's score is
 //    its largest c, or the sum of its two largest (group_fn), and only experts of the `keep_groups` best groups may be
 //    chosen (n_groups = 1: any; the others' c count as -inf); the `top` largest c are chosen (ties: the lower index),
-//    their weights are s / (sum of the chosen s + 1e-20) * weight_scale, or s * weight_scale without `normalize`.  The
+//    their weights are s / (sum of the chosen s + 1e-20) * weight_scale, or s * weight_scale without `normalize`.  A bias
+//    may be added to the logits first; with MOE_SCORE_LOGIT the choice goes by the logits themselves (+ correction) and
+//    the weights are the softmax of the chosen ones among themselves, * weight_scale.  The
 //    router may have more rows than there are experts with matrices: the rows behind those are identity experts,
 //    whose output is h_t itself; the kernels below skip them and the last one adds their share.  With w_sg (float [H]) it also
 //    gives sigmoid(w_sg . h), the gate of an expert that every token uses.
 //  * moe_gated_kernel: act[t, k, :] = act(Wg_e h_t) * (Wu_e h_t) for the k-th chosen expert e of token t (the
 //    nonlinearities of common.h: SiLU, or the clamped swish with its limit); the experts' gate and up rows are
 //    stacked: wgu [E, 2F, H], gate rows first.
+//  * moe_up_kernel: the same for experts without a gate, act[t, k, :] = act(Wu_e h_t); wu [E, F, H].
 //  * moe_down_kernel: out[t] = sum_k w[t, k] Wd_e act[t, k] (+ sg[t] * shared[t]); wd [E, H, F]; float out.  With a
 //    residual (Join) the layer's sum ends here: x[t] += out[t] + another result of the layer (float partial sums or
 //    one bf16 / float tensor, and a bias), in place, and x once more in the activations' type for a product that
@@ -22,7 +25,7 @@
 #include "common.h"
 
 #define MOE_MAX_EXPERTS 1024
-enum { MOE_SCORE_SOFTMAX = 0, MOE_SCORE_SIGMOID = 1 };
+enum { MOE_SCORE_SOFTMAX = 0, MOE_SCORE_SIGMOID = 1, MOE_SCORE_LOGIT = 2 };
 enum { MOE_GROUP_MAX = 0, MOE_GROUP_TOP2_SUM = 1 };
 
 // Where a layer's sum ends: the residual x [n, H], another result `a` to add (parts `stride` apart; may be absent) with
@@ -101,6 +104,7 @@ __global__ __launch_bounds__(256) void moe_logits_kernel(const T* __restrict__ h
 
 // grid (tokens), 64 threads: softmax, groups, the top choices and their weights from a row of logits
 __global__ __launch_bounds__(64) void moe_select_kernel(const float* __restrict__ logits,
+                                                        const float* __restrict__ bias,
                                                         const float* __restrict__ correction, int has_sg, int E,
                                                         int n_groups, int keep_groups, int top, int* __restrict__ idx_out,
                                                         float* __restrict__ w_out, float* __restrict__ sg_out,
@@ -114,27 +118,30 @@ __global__ __launch_bounds__(64) void moe_select_kernel(const float* __restrict_
     if (has_sg && lane == 0) sg_out[t] = 1.0f / (1.0f + expf(-zr[E]));
     if (score_fn == MOE_SCORE_SIGMOID) {
         for (int e = lane; e < E; e += 64) {
-            z[e] = 1.0f / (1.0f + expf(-zr[e]));
+            z[e] = 1.0f / (1.0f + expf(-(zr[e] + (bias ? bias[e] : 0.f))));
             c[e] = z[e] + (correction ? correction[e] : 0.f);
         }
     } else {
         float mx = -INFINITY;
         for (int e = lane; e < E; e += 64) {
-            z[e] = zr[e];
+            z[e] = zr[e] + (bias ? bias[e] : 0.f);
             mx = fmaxf(mx, z[e]);
         }
         mx = wave_max(mx);
         float sum = 0.f;
         for (int e = lane; e < E; e += 64) {
             const float p = expf(z[e] - mx);
+            if (score_fn == MOE_SCORE_LOGIT) c[e] = z[e] + (correction ? correction[e] : 0.f);
             z[e] = p;
             sum += p;
         }
-        sum = wave_sum(sum);
-        const float inv = 1.0f / sum;
-        for (int e = lane; e < E; e += 64) {
-            z[e] *= inv;
-            c[e] = z[e] + (correction ? correction[e] : 0.f);
+        if (score_fn == MOE_SCORE_SOFTMAX) {
+            sum = wave_sum(sum);
+            const float inv = 1.0f / sum;
+            for (int e = lane; e < E; e += 64) {
+                z[e] *= inv;
+                c[e] = z[e] + (correction ? correction[e] : 0.f);
+            }
         }
     }
     __builtin_amdgcn_wave_barrier();
@@ -193,12 +200,13 @@ __global__ __launch_bounds__(64) void moe_select_kernel(const float* __restrict_
     for (int r = lane; r < top; r += 64) w_out[t * top + r] *= norm;
 }
 
-extern "C" const char* cpmcu_moe_route(const void* h, long ldh, int dtype, const float* wr, const float* correction,
+extern "C" const char* cpmcu_moe_route(const void* h, long ldh, int dtype, const float* wr, const float* bias,
+                                       const float* correction,
                                        const float* w_sg, int n, int H, int E, int n_groups, int keep_groups, int top,
                                        float* logits, int* idx_out, float* w_out, float* sg_out, int score_fn,
                                        int group_fn, float weight_scale, int normalize, int logits_ready,
                                        hipStream_t stream) {
-    CPMCU_REQUIRE((score_fn == MOE_SCORE_SOFTMAX || score_fn == MOE_SCORE_SIGMOID) &&
+    CPMCU_REQUIRE((score_fn == MOE_SCORE_SOFTMAX || score_fn == MOE_SCORE_SIGMOID || score_fn == MOE_SCORE_LOGIT) &&
                   (group_fn == MOE_GROUP_MAX || group_fn == MOE_GROUP_TOP2_SUM),
                   "moe_route: unknown score function %d or group score %d", score_fn, group_fn);
     CPMCU_REQUIRE(n > 0 && H > 0 && E > 0 && logits, "moe_route: empty shape");
@@ -218,7 +226,7 @@ extern "C" const char* cpmcu_moe_route(const void* h, long ldh, int dtype, const
     else
         CPMCU_FAIL("moe_route: unknown dtype %d", dtype);
     CPMCU_LAUNCH_CHECK("moe_logits");
-    moe_select_kernel<<<n, 64, 0, stream>>>(logits, correction, w_sg ? 1 : 0, E, n_groups, keep_groups, top, idx_out, w_out,
+    moe_select_kernel<<<n, 64, 0, stream>>>(logits, bias, correction, w_sg ? 1 : 0, E, n_groups, keep_groups, top, idx_out, w_out,
                                             sg_out, score_fn, group_fn, weight_scale, normalize);
     CPMCU_LAUNCH_CHECK("moe_select");
     return nullptr;
@@ -266,6 +274,76 @@ extern "C" const char* cpmcu_moe_gated(const void* h, long ldh, int dtype, const
     else
         CPMCU_FAIL("moe_gated: unknown dtype %d", dtype);
     CPMCU_LAUNCH_CHECK("moe_gated");
+    return nullptr;
+}
+
+// grid (tokens * top, ceil(F / 16)), 256 threads: a wavefront takes 4 rows of the expert's F and reads them together,
+// against one piece of the token's row
+template <typename T>
+__global__ __launch_bounds__(256) void moe_up_kernel(const T* __restrict__ h, long ldh, const T* __restrict__ wu,
+                                                     const int* __restrict__ idx, T* __restrict__ act, int H, int F,
+                                                     int top, int E, int act_fn) {
+    const long pair = blockIdx.x;
+    const long t = pair / top;
+    const int e = idx[pair];
+    if (e >= E) return;                 // an identity expert
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int j0 = blockIdx.y * 4 * MOE_ROWS + wave * MOE_ROWS;
+    if (j0 >= F) return;
+    const T* hr = h + t * ldh;
+    const T* w = wu + (long)e * F * H;
+    const bool vec = (H % 8 == 0) && (ldh % 8 == 0) && ((uintptr_t)h % 32 == 0) && ((uintptr_t)wu % 32 == 0);
+    const T *w0 = w + (long)j0 * H, *w1 = w + (long)min(j0 + 1, F - 1) * H, *w2 = w + (long)min(j0 + 2, F - 1) * H,
+            *w3 = w + (long)min(j0 + 3, F - 1) * H;
+    float s0 = 0.f, s1 = 0.f, s2 = 0.f, s3 = 0.f;
+    if (vec) {
+#pragma unroll 2
+        for (int c = lane * 8; c < H; c += 64 * 8) {
+            float x[8], y0[8], y1[8], y2[8], y3[8];
+            load8<T>(w0 + c, y0);
+            load8<T>(w1 + c, y1);
+            load8<T>(w2 + c, y2);
+            load8<T>(w3 + c, y3);
+            load8<T>(hr + c, x);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                s0 += x[i] * y0[i];
+                s1 += x[i] * y1[i];
+                s2 += x[i] * y2[i];
+                s3 += x[i] * y3[i];
+            }
+        }
+    } else {
+        for (int c = lane; c < H; c += 64) {
+            const float x = to_f32(hr[c]);
+            s0 += x * to_f32(w0[c]);
+            s1 += x * to_f32(w1[c]);
+            s2 += x * to_f32(w2[c]);
+            s3 += x * to_f32(w3[c]);
+        }
+    }
+    s0 = wave_sum(s0);
+    s1 = wave_sum(s1);
+    s2 = wave_sum(s2);
+    s3 = wave_sum(s3);
+    if (lane < 4 && j0 + lane < F)
+        act[pair * F + j0 + lane] = from_f32<T>(plain_act(lane == 0 ? s0 : (lane == 1 ? s1 : (lane == 2 ? s2 : s3)), act_fn));
+}
+
+extern "C" const char* cpmcu_moe_up(const void* h, long ldh, int dtype, const void* wu, const int* idx, void* act, int n,
+                                    int H, int F, int top, int E, int act_fn, hipStream_t stream) {
+    CPMCU_REQUIRE(n > 0 && H > 0 && F > 0 && top > 0 && E > 0, "moe_up: empty shape");
+    CPMCU_REQUIRE(CPMCU_PLAIN_ACT_KNOWN(act_fn), "moe_up: unknown nonlinearity %d", act_fn);
+    const int fy = (F + 4 * MOE_ROWS - 1) / (4 * MOE_ROWS);
+    CPMCU_REQUIRE(fy <= 65535, "moe_up: %d rows an expert exceed the launch grid", F);
+    dim3 grid((unsigned)((long)n * top), fy);
+    if (dtype == CPMCU_F32)
+        moe_up_kernel<float><<<grid, 256, 0, stream>>>((const float*)h, ldh, (const float*)wu, idx, (float*)act, H, F, top, E, act_fn);
+    else if (dtype == CPMCU_BF16)
+        moe_up_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)h, ldh, (const bf16_t*)wu, idx, (bf16_t*)act, H, F, top, E, act_fn);
+    else
+        CPMCU_FAIL("moe_up: unknown dtype %d", dtype);
+    CPMCU_LAUNCH_CHECK("moe_up");
     return nullptr;
 }
 
@@ -400,6 +478,7 @@ extern "C" const char* cpmcu_moe_down(const void* act, int dtype, const void* wd
 //  * moe_gated_mfma_kernel: act[pair] = silu(Wg_e h_t) * (Wu_e h_t); a wavefront owns the 64 rows of a tile and 32
 //    features (two tiles of gate rows, two of up rows): 16 matrix instructions for 8 operand loads, operands
 //    straight from memory (the 4 wavefronts of a workgroup read the same rows of h, which meet in the CU's cache).
+//    Without a gate (GATED false; wgu then holds up rows only) it owns 64 features: act[pair] = act(Wu_e h_t).
 //  * moe_down_mfma_kernel: y[pair] = Wd_e act[pair] (bf16); a wavefront owns the 64 rows and 64 columns.
 //  * moe_combine_kernel: out[t] = sum_k w[t, k] y[t, k] (h_t where the chosen expert is an identity expert) (+ sg[t] * shared[t]) in float, k in order.
 // ===========================================================================
@@ -439,7 +518,9 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int* __restrict__
     }
 }
 
-// grid (ceil(F / 128), max_tiles), 256 threads: a wavefront takes all 64 rows of the tile and 32 features
+// grid (ceil(F / 128), or ceil(F / 256) without a gate, max_tiles), 256 threads: a wavefront takes all 64 rows of the tile
+// and 32 features (64 without a gate)
+template <bool GATED>
 __global__ __launch_bounds__(256) void moe_gated_mfma_kernel(const bf16_t* __restrict__ h, long ldh,
                                                              const bf16_t* __restrict__ wgu, const int* __restrict__ rows,
                                                              const int* __restrict__ tile_expert,
@@ -450,7 +531,7 @@ __global__ __launch_bounds__(256) void moe_gated_mfma_kernel(const bf16_t* __res
     const int wave = __builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));
     const int lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
     const int e = tile_expert[tile];
-    const int f0 = blockIdx.x * 128 + wave * 32;
+    const int f0 = GATED ? blockIdx.x * 128 + wave * 32 : blockIdx.x * 256 + wave * 64;
     if (f0 >= F) return;
     const bf16_t* xp[4];
 #pragma unroll
@@ -458,7 +539,7 @@ __global__ __launch_bounds__(256) void moe_gated_mfma_kernel(const bf16_t* __res
         const int pair = rows[tile * MOE_TILE + rt * 16 + r];
         xp[rt] = h + (long)(pair >= 0 ? pair / top : 0) * ldh + g * 8;
     }
-    const bf16_t* wp = wgu + (long)e * 2 * F * H + g * 8;
+    const bf16_t* wp = wgu + (long)e * (GATED ? 2 : 1) * F * H + g * 8;
     mfloatx4_t acc[4][4];
 #pragma unroll
     for (int rt = 0; rt < 4; ++rt)
@@ -467,8 +548,8 @@ __global__ __launch_bounds__(256) void moe_gated_mfma_kernel(const bf16_t* __res
     long wrow[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {                 // j = 0, 1: gate rows f0 + 16 j + r; j = 2, 3: their up rows
-        const int f = min(f0 + 16 * (j & 1) + r, F - 1);
-        wrow[j] = (long)((j >> 1) * F + f) * H;
+        const int f = min(f0 + 16 * (GATED ? (j & 1) : j) + r, F - 1);
+        wrow[j] = (long)((GATED ? (j >> 1) * F : 0) + f) * H;
     }
     for (int k0 = 0; k0 < H; k0 += 32) {
         const bool k_ok = k0 + g * 8 < H;
@@ -495,12 +576,16 @@ __global__ __launch_bounds__(256) void moe_gated_mfma_kernel(const bf16_t* __res
             const int p = rows[tile * MOE_TILE + rt * 16 + 4 * g + i];
             if (p < 0) continue;
 #pragma unroll
-            for (int j = 0; j < 2; ++j) {
+            for (int j = 0; j < (GATED ? 2 : 4); ++j) {
                 const int f = f0 + 16 * j + r;
                 if (f < F) {
-                    float gt = acc[rt][j][i], up = acc[rt][2 + j][i];
-                    gate_prepare(gt, up, act_fn, act_limit);
-                    act[(long)p * F + f] = f32_to_bf16(gate_act(gt, act_fn) * up);
+                    if (GATED) {
+                        float gt = acc[rt][j][i], up = acc[rt][(2 + j) & 3][i];
+                        gate_prepare(gt, up, act_fn, act_limit);
+                        act[(long)p * F + f] = f32_to_bf16(gate_act(gt, act_fn) * up);
+                    } else {
+                        act[(long)p * F + f] = f32_to_bf16(plain_act(acc[rt][j][i], act_fn));
+                    }
                 }
             }
         }
@@ -622,13 +707,13 @@ extern "C" const char* cpmcu_moe_experts_mfma(const void* h, long ldh, const voi
                                               const float* w, const void* shared, int shared_dtype, int shared_parts,
                                               long shared_stride, const float* sg, void* act, void* y, int* rows,
                                               int* tile_expert, int* n_tiles, int max_tiles, float* out, int n, int H,
-                                              int F, int E, int top, int act_fn, float act_limit, float* x, const void* a,
+                                              int F, int E, int top, int gated, int act_fn, float act_limit, float* x, const void* a,
                                               int a_dtype, int a_parts, long a_stride, const float* a_bias, void* copy,
                                               hipStream_t stream) {
     const Join join{x, a, a_dtype == CPMCU_BF16, a ? a_parts : 0, a_stride, a_bias, copy};
     if (const char* m = join_check(join, out)) return m;
     CPMCU_REQUIRE(n > 0 && H > 0 && F > 0 && E > 0 && top > 0, "moe_experts_mfma: empty shape");
-    CPMCU_REQUIRE(CPMCU_ACT_KNOWN(act_fn), "moe_experts_mfma: unknown nonlinearity %d", act_fn);
+    CPMCU_REQUIRE(gated ? CPMCU_ACT_KNOWN(act_fn) : CPMCU_PLAIN_ACT_KNOWN(act_fn), "moe_experts_mfma: unknown nonlinearity %d", act_fn);
     CPMCU_REQUIRE(E <= MOE_MAX_EXPERTS, "moe_experts_mfma: %d experts (up to %d are taken)", E, MOE_MAX_EXPERTS);
     CPMCU_REQUIRE(H % 8 == 0 && F % 8 == 0 && ldh % 8 == 0 && (uintptr_t)h % 16 == 0 && (uintptr_t)wgu % 16 == 0 &&
                   (uintptr_t)wd % 16 == 0 && (uintptr_t)act % 16 == 0,
@@ -638,8 +723,12 @@ extern "C" const char* cpmcu_moe_experts_mfma(const void* h, long ldh, const voi
                   "moe_experts_mfma: %d tiles of scratch for %ld pairs of %d experts (at most 65535)", max_tiles, pairs, E);
     moe_group_kernel<<<1, 1024, 0, stream>>>(idx, (int)pairs, E, rows, tile_expert, n_tiles, max_tiles);
     CPMCU_LAUNCH_CHECK("moe_group");
-    moe_gated_mfma_kernel<<<dim3((F + 127) / 128, max_tiles), 256, 0, stream>>>((const bf16_t*)h, ldh, (const bf16_t*)wgu, rows,
-                                                                            tile_expert, n_tiles, (bf16_t*)act, H, F, top, act_fn, act_limit);
+    if (gated)
+        moe_gated_mfma_kernel<true><<<dim3((F + 127) / 128, max_tiles), 256, 0, stream>>>(
+            (const bf16_t*)h, ldh, (const bf16_t*)wgu, rows, tile_expert, n_tiles, (bf16_t*)act, H, F, top, act_fn, act_limit);
+    else
+        moe_gated_mfma_kernel<false><<<dim3((F + 255) / 256, max_tiles), 256, 0, stream>>>(
+            (const bf16_t*)h, ldh, (const bf16_t*)wgu, rows, tile_expert, n_tiles, (bf16_t*)act, H, F, top, act_fn, act_limit);
     CPMCU_LAUNCH_CHECK("moe_gated_mfma");
     moe_down_mfma_kernel<<<dim3((H + 255) / 256, max_tiles), 256, 0, stream>>>((const bf16_t*)act, (const bf16_t*)wd, rows,
                                                                            tile_expert, n_tiles, (bf16_t*)y, H, F);

@@ -247,7 +247,7 @@ class Engine:
                      options: Optional[EngineOptions] = None) -> "Engine":
         options = options or EngineOptions()
         arch = get_architecture(config.architecture)
-        model = arch.build_model(config, options.model_options, tensors.keys())
+        model = arch.build_model(config, options.model_options, {k: tuple(v.shape) for k, v in tensors.items()})
         from ..weights.loader import _compare
         _compare(model.all_weight_specs(), {k: tuple(v.shape) for k, v in tensors.items()}, "the given tensors")
         dev = torch.device(options.device)

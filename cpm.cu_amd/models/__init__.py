@@ -6,3 +6,4 @@ from . import gumodra
 from . import sagedra
 from . import nelutar
 from . import pemalorn
+from . import tirizen

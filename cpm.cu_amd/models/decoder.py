@@ -18,7 +18,6 @@ from typing import List, Optional, Sequence
 
 import torch
 
-from .. import ops
 from ..cache.paged import CacheNeeds
 from ..parts.base import Block, Norm, Part, ResidualStream, Runtime, StepContext, branch_for
 from ..parts.embedding import LMHead, TokenEmbedding
@@ -98,14 +97,11 @@ class DecoderModel(Part):
     def forward(self, ctx: StepContext) -> torch.Tensor:
         """float32 logits [R, V] at ctx.logit_rows; the step's tokens enter the cache."""
         with ctx.timed("embed"):
+            kw = {"streams": self.streams} if self.streams else {}
             if self.embedding_entry is not None:
-                x = self.embedding.forward(ctx, ctx.cache.view(self.embedding_entry))
+                x = self.embedding.forward(ctx, ctx.cache.view(self.embedding_entry), **kw)
             else:
-                x = self.embedding.forward(ctx)
-            if self.streams:
-                lanes = ctx.ws.get("residual.streams", (self.streams,) + tuple(x.shape), torch.float32)
-                ops.streams_fill(x, lanes)
-                x = lanes
+                x = self.embedding.forward(ctx, **kw)
             if self.loop_input is not None:
                 self.loop_input.start(x, ctx)
             stream = ResidualStream(x)

@@ -72,15 +72,26 @@ def _check(msg):
 
 
 # ---------------------------------------------------------------------------
-def embed(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor, scale: float):
-    """out[r] = float(table[ids[r]]) * scale;  table [V,H], ids int32 [n], out float32 [n,H]."""
+def embed(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor, scale: float,
+          pos_table: Optional[torch.Tensor] = None, positions: Optional[torch.Tensor] = None):
+    """out[r] = float(table[ids[r]]) * scale (+ float(pos_table[positions[r]]), a learned vector a position; pos_table
+    [P, H] of the table's type, positions int32 [n] below P);  table [V,H], ids int32 [n], out float32 [n,H], or
+    [S,n,H] for S equal copies (the streams of a residual at their start)."""
     _need(table, "embed table", shape=(None, None))
     V, H = table.shape
     _need(ids, "embed ids", torch.int32, (None,))
     n = ids.shape[0]
-    _need(out, "embed out", torch.float32, (n, H))
+    copies = 1
+    if out.dim() == 3:
+        copies = out.shape[0]
+        _need(out, "embed out", torch.float32, (None, n, H))
+    else:
+        _need(out, "embed out", torch.float32, (n, H))
+    if pos_table is not None:
+        _need(pos_table, "embed position table", table.dtype, (None, H))
+        _need(positions, "embed positions", torch.int32, (n,))
     _check(_fn("core", "cpmcu_embed")(_p(table), c_int(_code(table)), _p(ids), _p(out), c_int(n), c_int(H), c_int(V),
-                                      c_float(scale), _stream()))
+                                      c_float(scale), _p(pos_table), _p(positions), c_int(copies), _stream()))
 
 
 def add_rms_norm(x: torch.Tensor, branch: Optional[torch.Tensor], branch_scale: float, weight: torch.Tensor,
@@ -191,6 +202,23 @@ def _act(activation):
     """(c_int code, c_float limit) for the kernels."""
     name, limit = gate_activation(activation)
     return c_int(GATE_ACTIVATIONS[name]), c_float(limit)
+
+
+PLAIN_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "relu_squared": 3}
+
+
+def plain_activation(name: str) -> str:
+    """The nonlinearity of a feed-forward without a gate: 'silu', 'gelu_tanh' or 'relu_squared' (max(z, 0)^2)."""
+    if name not in PLAIN_ACTIVATIONS:
+        raise KernelError(f"nonlinearity '{name}' is not supported without a gate ({sorted(PLAIN_ACTIVATIONS)})")
+    return name
+
+
+def activate(z: torch.Tensor, activation: str):
+    """z <- act(z) in place (plain_activation)."""
+    _need(z, "activation input")
+    _check(_fn("core", "cpmcu_activate")(_p(z), c_int(_code(z)), c_long(z.numel()), c_int(PLAIN_ACTIVATIONS[plain_activation(activation)]),
+                                         _stream()))
 
 
 def silu_mul(gate_up: torch.Tensor, out: torch.Tensor, activation="silu"):
@@ -688,14 +716,14 @@ def qkv_norm_rotate_store(qkv: torch.Tensor, q_out: torch.Tensor, nh: int, nkv: 
                           bias: Optional[torch.Tensor] = None, q_norm: Optional[torch.Tensor] = None,
                           k_norm: Optional[torch.Tensor] = None, eps: float = 0.0, values_from_keys: bool = False,
                           norm_after: bool = False, interleaved: bool = False, q_scale: Optional[torch.Tensor] = None,
-                          v_inv_freq: Optional[torch.Tensor] = None):
+                          v_inv_freq: Optional[torch.Tensor] = None, temp_coef: float = 0.0, temp_every: int = 0):
     """qkv_rotate_store with what some designs put between projection and rotation: ``bias`` (float32, as wide as
     a row of qkv) is added; q heads and k heads are divided by their root mean square (eps inside the root) and
     multiplied by a weight of dk numbers shared by the heads (q_norm, k_norm, float32 [dk]); with
     values_from_keys a row is [q | k] only and the value pages receive k as projected (with its bias, before norm
     and rotation).  With norm_after the q and k heads are rotated first and then divided by their root mean square
     (times q_norm / k_norm where given, by nothing else where not).  ``interleaved`` as in qkv_rotate_store.
-    q_scale (float32 [nh]) multiplies a finished query head; v_inv_freq (float32 [dv/2]): value heads are rotated by
+    q_scale (float32 [nh]) multiplies a finished query head, and so does the temperature of qkv_row_norm_store; v_inv_freq (float32 [dv/2]): value heads are rotated by
     their positions as well, over all dv features (head_output turns what the attention makes of them back).  The
     rows of qkv may be float32 where q_out and the cache are bfloat16 (rows that a convolution wrote)."""
     ld = _ld(qkv, "qkv")
@@ -739,7 +767,58 @@ def qkv_norm_rotate_store(qkv: torch.Tensor, q_out: torch.Tensor, nh: int, nkv: 
         _p(tok_slot), _p(inv_freq), c_float(mag), _p(kpool if write_kv else None), _p(vpool if write_kv else None),
         _p(page_table if write_kv else None), c_int(tw), c_int(page_size), c_int(pk), c_int(pv),
         c_int(1 if write_kv else 0), c_int(1 if norm_after else 0), c_int(1 if interleaved else 0), c_int(_code(qkv)),
-        _p(q_scale), _p(v_inv_freq), _stream()))
+        _p(q_scale), _p(v_inv_freq), c_float(temp_coef), c_int(temp_every), _stream()))
+
+
+QKV_ROW_MAX = 15360       # features of the widest projection that qkv_row_norm_store norms as a whole
+
+
+def qkv_row_norm_store(qkv: torch.Tensor, q_out: torch.Tensor, nh: int, nkv: int, dk: int, dv: int, rot_dims: int,
+                       positions: torch.Tensor, tok_slot: torch.Tensor, inv_freq: Optional[torch.Tensor], mag: float,
+                       kpool: Optional[torch.Tensor], vpool: Optional[torch.Tensor], page_table: Optional[torch.Tensor],
+                       page_size: int, q_norm: torch.Tensor, k_norm: Optional[torch.Tensor], eps: float, write_kv: bool = True,
+                       temp_coef: float = 0.0, temp_every: int = 0, interleaved: bool = False, gate_col: int = 0,
+                       gate_out: Optional[torch.Tensor] = None):
+    """qkv_rotate_store for designs that norm a whole projection at once: the nh*dk query numbers of a row are divided by
+    their root mean square (eps inside the root) and multiplied by q_norm (float32 [nh*dk]), the nkv*dk key numbers
+    likewise by k_norm, before heads are split and rotated.  Finished queries are multiplied by
+    1 + temp_coef ln(floor((p + 1) / temp_every) + 1) (temp_every 0: not).  qkv [n, W], or float32 partial sums [S, n, W]
+    of a split product.  gate_out [n, nh] (q_out's type): the nh numbers of a row from column gate_col on, copied."""
+    nparts, stride, src = 1, 0, qkv
+    if qkv.dim() == 3:
+        _need(qkv, "qkv partial sums", torch.float32, (None, None, None))
+        nparts, stride, src = qkv.shape[0], qkv.shape[1] * qkv.shape[2], qkv[0]
+    ld = _ld(src, "qkv")
+    n = src.shape[0]
+    width = nh * dk + (nkv * (dk + dv) if write_kv else 0)
+    if src.shape[1] < width or (gate_out is not None and (gate_col < width or src.shape[1] < gate_col + nh)):
+        raise KernelError(f"qkv_row_norm_store: rows of {src.shape[1]} cannot hold {nh} query heads, {nkv} key/value heads and their gates")
+    _need(q_out, "qkv q_out", shape=(n, nh * dk))
+    if src.dtype != q_out.dtype and src.dtype != torch.float32:
+        raise KernelError(f"qkv_row_norm_store: rows of {src.dtype} for outputs of {q_out.dtype}")
+    _need(positions, "qkv positions", torch.int32, (n,))
+    if rot_dims:
+        _need(inv_freq, "qkv inv_freq", torch.float32, (rot_dims // 2,))
+    _need(q_norm, "qkv query norm weight", torch.float32, (nh * dk,))
+    if gate_out is not None:
+        _need(gate_out, "qkv head gates", q_out.dtype, (n, nh))
+    tw = pk = pv = 0
+    if write_kv:
+        _need(k_norm, "qkv key norm weight", torch.float32, (nkv * dk,))
+        _need(tok_slot, "qkv token slots", torch.int32, (n,))
+        _need(page_table, "qkv page table", torch.int32, (None, None))
+        _need(kpool, "qkv key pool", q_out.dtype, (None, page_size, None))
+        _need(vpool, "qkv value pool", q_out.dtype, (kpool.shape[0], page_size, None))
+        if kpool.shape[2] % nkv or vpool.shape[2] % nkv:
+            raise KernelError(f"qkv_row_norm_store: pools of {kpool.shape[2]} / {vpool.shape[2]} features do not hold {nkv} heads")
+        tw, pk, pv = page_table.shape[1], kpool.shape[2] // nkv, vpool.shape[2] // nkv
+    _check(_fn("attention_general", "cpmcu_qkv_row_norm_store")(
+        _p(src), c_int(_code(src)), c_long(ld), c_int(nparts), c_long(stride), _p(q_out), c_int(_code(q_out)), c_int(n), c_int(nh),
+        c_int(nkv), c_int(dk), c_int(dv), c_int(rot_dims), _p(q_norm), _p(k_norm if write_kv else None), c_float(eps),
+        c_float(temp_coef), c_int(temp_every), _p(positions), _p(tok_slot), _p(inv_freq), c_float(mag),
+        _p(kpool if write_kv else None), _p(vpool if write_kv else None), _p(page_table if write_kv else None), c_int(tw),
+        c_int(page_size), c_int(pk), c_int(pv), c_int(1 if write_kv else 0), c_int(1 if interleaved else 0), c_long(gate_col),
+        _p(gate_out), _stream()))
 
 
 def _parts_of(t: torch.Tensor, n: int, H: int, name: str):
@@ -1150,6 +1229,103 @@ def delta_scan(qkv: torch.Tensor, gates: Optional[torch.Tensor], a_off: int, b_o
 DELTA_RULES = {"delta": 0, "channel": 1, "decay": 2}
 
 
+GLA_SEGMENT = 64          # a segment is a multiple of so many tokens
+
+
+def gla_segments(q_lens: Sequence[int], heads: int, dv: int) -> Tuple[int, int]:
+    """(segments a sequence, tokens a segment) for gla_scan: a walk over a few long sequences leaves most of the chip idle,
+    so they are cut into segments that run at the same time until there are about eight workgroups a compute unit.  (1, 0):
+    not cut."""
+    longest = max(q_lens)
+    wgs = len(q_lens) * heads * (-(-dv // 32))
+    want = min(max(8 * compute_units() // wgs, 1), longest // (2 * GLA_SEGMENT))
+    if want <= 1:
+        return 1, 0
+    seg = -(-(-(-longest // want)) // GLA_SEGMENT) * GLA_SEGMENT
+    n = -(-longest // seg)
+    return (n, seg) if n > 1 else (1, 0)
+
+
+def gla_segment_rows(max_step_tokens: int, heads: int, dv: int) -> int:
+    """The most (sequence, segment) pairs that gla_segments makes of a step (0: it cuts none)."""
+    if max_step_tokens < 4 * GLA_SEGMENT:
+        return 0
+    return max(8 * compute_units() // (heads * -(-dv // 32)), 0)
+
+
+def channel_decay(low: torch.Tensor, up: torch.Tensor, bias: torch.Tensor, tau: float, out: torch.Tensor):
+    """out = sigmoid(low . up + bias)^(1/tau), float32 [n, C]: low [n, R] (may be a column slice), up float32 [R, C] (the
+    transpose of a checkpoint's second half), bias float32 [C]."""
+    ld = _ld(low, "decay input")
+    n, R = low.shape
+    _need(up, "decay product", torch.float32, (R, None))
+    C = up.shape[1]
+    _need(bias, "decay bias", torch.float32, (C,))
+    _need(out, "decays", torch.float32, (n, C))
+    if not tau > 0:
+        raise KernelError(f"channel_decay: tau {tau}")
+    _check(_fn("gla", "cpmcu_channel_decay")(_p(low), c_int(_code(low)), c_long(ld), c_int(R), _p(up), _p(bias), c_float(1.0 / tau),
+                                             _p(out), c_int(n), c_int(C), _stream()))
+
+
+def gla_scan(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: torch.Tensor, state: torch.Tensor, y: torch.Tensor,
+             cu_q: torch.Tensor, seq_slot: torch.Tensor, heads: int, dk: int, dv: int, q_scale: float, segments: int = 1,
+             seg_len: int = 0, scratch: Optional[Sequence[torch.Tensor]] = None):
+    """Linear attention whose decay is a number a head and key channel, over each sequence's tokens, in float:
+    S <- diag(decay_t) S + k v^T, y = S^T (q_scale q).  rows [n, W] holds q and k heads at columns q_off and k_off (heads x
+    dk each) and v heads at v_off (heads x dv); decay float32 [n, heads*dk]; state float32 [slots, heads, dv, dk]; y float32
+    [n, heads*dv].  segments > 1: every sequence is cut into that many pieces of seg_len tokens, which run at the same time
+    (gla_segments); scratch then holds float32 [B * segments, heads, dv, dk], [B * segments, heads, dk] and [n, heads*dk]."""
+    ld = _ld(rows, "gla rows")
+    n = rows.shape[0]
+    if min(q_off, k_off, v_off) < 0 or max(q_off + heads * dk, k_off + heads * dk, v_off + heads * dv) > rows.shape[1]:
+        raise KernelError(f"gla_scan: columns beyond rows of {tuple(rows.shape)}")
+    _need(decay, "gla decays", torch.float32, (n, heads * dk))
+    _need(state, "gla state", torch.float32, (None, heads, dv, dk))
+    _need(y, "gla out", torch.float32, (n, heads * dv))
+    _need(cu_q, "gla sequence starts", torch.int32, (None,))
+    B = cu_q.shape[0] - 1
+    _need(seq_slot, "gla sequence slots", torch.int32, (B,))
+    ss = sd = qa = None
+    if segments > 1:
+        ss, sd, qa = scratch
+        _need(ss, "gla segment states", torch.float32, (B * segments, heads, dv, dk))
+        _need(sd, "gla segment decays", torch.float32, (B * segments, heads, dk))
+        _need(qa, "gla decayed queries", torch.float32, (n, heads * dk))
+    _check(_fn("gla", "cpmcu_gla_scan")(_p(rows), c_int(_code(rows)), c_long(ld), c_long(q_off), c_long(k_off), c_long(v_off),
+                                        _p(decay), _p(state), _p(y), _p(cu_q), _p(seq_slot), c_int(B), c_int(heads), c_int(dk),
+                                        c_int(dv), c_float(q_scale), c_int(segments), c_int(seg_len), _p(ss), _p(sd), _p(qa),
+                                        _stream()))
+
+
+def gla_step(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, g_off: int, low_off: int, up: torch.Tensor,
+             bias: torch.Tensor, tau: float, norm_w: torch.Tensor, eps: float, state: torch.Tensor, out: torch.Tensor,
+             cu_q: torch.Tensor, seq_slot: torch.Tensor, heads: int, dk: int, dv: int, q_scale: float,
+             gate_activation: str = "silu"):
+    """A step of one token a sequence in one launch: channel_decay of columns low_off.., one step of gla_scan, each head
+    divided by its root mean square (eps inside the root) and multiplied by norm_w (float32 [dv], shared by the heads) and by
+    silu (or sigmoid) of the gate at g_off (heads x dv); out [n, heads*dv] of rows' type."""
+    ld = _ld(rows, "gla rows")
+    n = rows.shape[0]
+    R = up.shape[0]
+    _need(up, "decay product", torch.float32, (R, heads * dk))
+    _need(bias, "decay bias", torch.float32, (heads * dk,))
+    _need(norm_w, "gla norm weight", torch.float32, (dv,))
+    if min(q_off, k_off, v_off, g_off, low_off) < 0 or rows.shape[1] < max(q_off + heads * dk, k_off + heads * dk, v_off + heads * dv,
+                                                                           g_off + heads * dv, low_off + R):
+        raise KernelError(f"gla_step: columns beyond rows of {tuple(rows.shape)}")
+    _need(state, "gla state", torch.float32, (None, heads, dv, dk))
+    _need(out, "gla out", rows.dtype, (n, heads * dv))
+    _need(cu_q, "gla sequence starts", torch.int32, (n + 1,))
+    _need(seq_slot, "gla sequence slots", torch.int32, (n,))
+    if not tau > 0 or gate_activation not in ("silu", "sigmoid"):
+        raise KernelError(f"gla_step: tau {tau}, gate nonlinearity '{gate_activation}'")
+    _check(_fn("gla", "cpmcu_gla_step")(_p(rows), c_int(_code(rows)), c_long(ld), c_long(q_off), c_long(k_off), c_long(v_off),
+                                        c_long(g_off), c_long(low_off), c_int(R), _p(up), _p(bias), c_float(1.0 / tau), _p(norm_w),
+                                        c_float(eps), c_int(1 if gate_activation == "sigmoid" else 0), _p(state), _p(out), _p(cu_q),
+                                        _p(seq_slot), c_int(n), c_int(heads), c_int(dk), c_int(dv), c_float(q_scale), _stream()))
+
+
 def linear_attention_prepare(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, out: torch.Tensor, heads: int,
                              dk: int, dv: int, silu: bool, positions: Optional[torch.Tensor] = None,
                              inv_freq: Optional[torch.Tensor] = None, interleaved: bool = False, k_scale: float = 1.0):
@@ -1220,7 +1396,7 @@ def diff_combine(a: torch.Tensor, out: torch.Tensor, heads: int, kv_heads: int, 
 
 
 MOE_MAX_EXPERTS = 1024
-MOE_SCORES = {"softmax": 0, "sigmoid": 1}
+MOE_SCORES = {"softmax": 0, "sigmoid": 1, "logit": 2}
 MOE_GROUP_SCORES = {"max": 0, "top2_sum": 1}
 
 
@@ -1228,13 +1404,15 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.
               n_groups: int, keep_groups: int, top: int, idx: torch.Tensor, weights: torch.Tensor,
               shared_out: Optional[torch.Tensor] = None, logits: Optional[torch.Tensor] = None,
               score: str = "softmax", group_score: str = "max", weight_scale: float = 1.0, normalize: bool = True,
-              logits_ready: bool = False):
+              logits_ready: bool = False, bias: Optional[torch.Tensor] = None):
     """Routing of every token to ``top`` of E experts.  Logits router . h in float (router float32 [E, H]), scores
     s = softmax over the experts (``score`` 'sigmoid': of each logit alone); choice scores s + correction; the
     experts form n_groups equal groups of neighbours, of which only the keep_groups with the largest group score may
     be chosen from (``group_score`` 'max': a group's best choice score; 'top2_sum': the sum of its two best); the top
     largest choice scores win (ties: the lower index); weights = s of the chosen / (their sum + 1e-20) *
-    weight_scale (without ``normalize`` s * weight_scale).  idx int32 [n, top], weights float32 [n, top].
+    weight_scale (without ``normalize`` s * weight_scale).  ``score`` 'logit': the choice goes by the logits (+ correction)
+    and the weights are the softmax of the chosen logits among themselves.  bias (float32 [E]) is added to the logits
+    first, for choice and weights.  idx int32 [n, top], weights float32 [n, top].
     shared_gate (float32 [H]): shared_out[t] = sigmoid(shared_gate . h[t]).  logits: float32 [n, E + 1] of scratch
     (allocated here when absent: a caller that must not allocate brings it); with logits_ready it holds the products
     (the shared gate's in column E) already."""
@@ -1254,10 +1432,14 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.
     if logits is None:
         logits = torch.empty((n, E + 1), dtype=torch.float32, device=h.device)
     _need(logits, "router logits", torch.float32, (n, E + 1))
+    if bias is not None:
+        _need(bias, "router bias", torch.float32, (E,))
+    if score == "logit" and not normalize:
+        raise KernelError("moe_route: weights that are a softmax of the chosen logits are normalised")
     if score not in MOE_SCORES or group_score not in MOE_GROUP_SCORES:
         raise KernelError(f"moe_route: score '{score}' ({sorted(MOE_SCORES)}) or group score '{group_score}' "
                           f"({sorted(MOE_GROUP_SCORES)}) is not known")
-    _check(_fn("moe", "cpmcu_moe_route")(_p(h), c_long(ldh), c_int(_code(h)), _p(router), _p(correction), _p(shared_gate),
+    _check(_fn("moe", "cpmcu_moe_route")(_p(h), c_long(ldh), c_int(_code(h)), _p(router), _p(bias), _p(correction), _p(shared_gate),
                                          c_int(n), c_int(H), c_int(E), c_int(n_groups), c_int(keep_groups), c_int(top),
                                          _p(logits), _p(idx), _p(weights), _p(shared_out), c_int(MOE_SCORES[score]),
                                          c_int(MOE_GROUP_SCORES[group_score]), c_float(weight_scale), c_int(1 if normalize else 0),
@@ -1279,6 +1461,19 @@ def moe_gated(h: torch.Tensor, gate_up: torch.Tensor, idx: torch.Tensor, act: to
     _need(act, "experts act", h.dtype, (n, top, F2 // 2))
     _check(_fn("moe", "cpmcu_moe_gated")(_p(h), c_long(ldh), c_int(_code(h)), _p(gate_up), _p(idx), _p(act), c_int(n),
                                          c_int(H), c_int(F2 // 2), c_int(top), c_int(E), *_act(activation), _stream()))
+
+
+def moe_up(h: torch.Tensor, up: torch.Tensor, idx: torch.Tensor, act: torch.Tensor, activation: str):
+    """moe_gated for experts without a gate: act[t, k] = act(Wu_e h[t]) (plain_activation), up [E, F, H]."""
+    ldh = _ld(h, "experts input")
+    n, H = h.shape
+    _need(up, "experts up", h.dtype, (None, None, H))
+    E, F = up.shape[0], up.shape[1]
+    _need(idx, "chosen experts", torch.int32, (n, None))
+    top = idx.shape[1]
+    _need(act, "experts act", h.dtype, (n, top, F))
+    _check(_fn("moe", "cpmcu_moe_up")(_p(h), c_long(ldh), c_int(_code(h)), _p(up), _p(idx), _p(act), c_int(n), c_int(H), c_int(F),
+                                      c_int(top), c_int(E), c_int(PLAIN_ACTIVATIONS[plain_activation(activation)]), _stream()))
 
 
 class Join:
@@ -1354,14 +1549,15 @@ def moe_experts_mfma_ok(h: torch.Tensor, expert_size: int, n_tiles: int) -> bool
 def moe_experts_mfma(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, idx: torch.Tensor, weights: torch.Tensor,
                      out: Optional[torch.Tensor], act: torch.Tensor, y: torch.Tensor, rows: torch.Tensor, tile_expert: torch.Tensor,
                      n_tiles: torch.Tensor, shared: Optional[torch.Tensor] = None,
-                     shared_gate: Optional[torch.Tensor] = None, activation="silu", join: Optional[Join] = None):
-    """moe_gated + moe_down for steps of many tokens, bf16 on the matrix cores: the (token, expert) pairs are grouped
+                     shared_gate: Optional[torch.Tensor] = None, activation="silu", join: Optional[Join] = None,
+                     gated: bool = True):
+    """moe_gated (without ``gated`` moe_up; gate_up is then [E, F, H]) + moe_down for steps of many tokens, bf16 on the matrix cores: the (token, expert) pairs are grouped
     by expert into tiles of MOE_TILE rows (pairs of identity experts, idx >= E, have none: they add h).  Scratch: act bf16 [n, top, F], y bf16 [n, top, H], rows int32
     [tiles * MOE_TILE], tile_expert int32 [tiles], n_tiles int32 [1], tiles >= moe_tiles(n, top, E)."""
     ldh = _ld(h, "experts input")
     n, H = h.shape
     _need(gate_up, "experts gate/up", torch.bfloat16, (None, None, H))
-    E, F = gate_up.shape[0], gate_up.shape[1] // 2
+    E, F = gate_up.shape[0], gate_up.shape[1] // (2 if gated else 1)
     _need(down, "experts down", torch.bfloat16, (E, H, F))
     _need(idx, "chosen experts", torch.int32, (n, None))
     top = idx.shape[1]
@@ -1383,7 +1579,8 @@ def moe_experts_mfma(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
         _p(h), c_long(ldh), _p(gate_up), _p(down), _p(idx), _p(weights), _p(shared),
         c_int(_code(shared) if shared is not None else 0), c_int(sp), c_long(sstr), _p(shared_gate), _p(act), _p(y),
         _p(rows), _p(tile_expert), _p(n_tiles), c_int(tiles), _p(out), c_int(n), c_int(H), c_int(F), c_int(E), c_int(top),
-        *_act(activation), *_join_args(join, n, H, torch.bfloat16), _stream()))
+        c_int(1 if gated else 0), *(_act(activation) if gated else (c_int(PLAIN_ACTIVATIONS[plain_activation(activation)]), c_float(0.0))),
+        *_join_args(join, n, H, torch.bfloat16), _stream()))
 
 
 def latent_store(q_out: Optional[torch.Tensor], nh: int, dim: int, rot: int, rank: int, eps: float, positions: torch.Tensor,
@@ -1721,7 +1918,7 @@ def gemm_skinny(x: torch.Tensor, w, out: torch.Tensor, alpha: float = 1.0, mode:
                 row_scale: Optional[RowScale] = None, activation="silu"):
     """bf16 product for at most 64 rows of x on the matrix cores, streaming w once; w is [N, K] as in the
     checkpoint or a TiledWeight.
-    mode 'plain': out [m,N] float32 or bfloat16; 'partial': out float32 [S,m,N], S slices of K to be summed by
+    mode 'plain': out [m,N] float32 or bfloat16; 'act': out bfloat16 [m,N] = act(product) (plain_activation); 'partial': out float32 [S,m,N], S slices of K to be summed by
     the consumer; 'gated': w holds gate rows then up rows, out bfloat16 [m,N/2] = act(gate) * up (act as in silu_mul).
     With row_scale, x is the x * w of add_norm_columns: the rows of the product are multiplied by the norm's
     factor (before the gate's nonlinearity)."""
@@ -1747,6 +1944,9 @@ def gemm_skinny(x: torch.Tensor, w, out: torch.Tensor, alpha: float = 1.0, mode:
     elif mode == "gated":
         _need(out, "gemm gated out", torch.bfloat16, (M, N // 2))
         omode, ldy = 2, N // 2
+    elif mode == "act":
+        _need(out, "gemm activated out", torch.bfloat16, (M, N))
+        omode, ldy = 3, N
     else:
         raise KernelError(f"gemm_skinny: unknown mode '{mode}'")
     _check(_fn("gemm", "cpmcu_gemm_skinny")(_p(x), c_long(K), _p(wt), c_long(K), _p(out), c_long(ldy),
@@ -1755,7 +1955,8 @@ def gemm_skinny(x: torch.Tensor, w, out: torch.Tensor, alpha: float = 1.0, mode:
                                             _p(row_scale.sums if row_scale is not None else None),
                                             c_int(row_scale.sums.shape[1] if row_scale is not None else 0),
                                             c_float(row_scale.eps if row_scale is not None else 0.0),
-                                            *_act(activation), _stream()))
+                                            *((c_int(PLAIN_ACTIVATIONS[plain_activation(activation)]), c_float(0.0))
+                                              if mode == "act" else _act(activation)), _stream()))
 
 
 SKINNY_MAX_ROWS = 64

@@ -11,8 +11,8 @@ from .mlstm import MLSTMMixer
 from .diff_attention import DifferentialAttention
 from .delta import GatedDeltaMixer
 from .parallel import ParallelMixer
-from .linear_attention import DecayLinearAttention
-from .ffn import GatedFFN, PolyNormFFN, RoutedExpertsFFN
+from .linear_attention import DecayLinearAttention, GatedLinearAttention
+from .ffn import GatedFFN, PlainFFN, PolyNormFFN, RoutedExpertsFFN
 from .input_conv import InputConvolution
 from .token_input import TokenInput, TokenTable
 from .loop_input import LoopInput

@@ -17,7 +17,7 @@ compressed key j is visible iff kernel_stride*j + kernel_size <= p.
 """
 from __future__ import annotations
 
-from typing import List, Mapping, Optional
+from typing import List, Mapping, Optional, Tuple
 
 import torch
 
@@ -254,6 +254,11 @@ class GeneralAttention(Mixer):
     'interleaved': 2i with 2i + 1).
     ``value_position``: a rotation of all value features (no magnitude, the pairs of ``position``): the value of key j is
     cached rotated by j, and a head's output at position p is turned back by p, before any gate.
+    ``norm_rows``: 'q_norm' and 'k_norm' hold as many numbers as the projections, and all query heads of a token are
+    divided by one root mean square, as are all its key heads (before heads are split and rotated).
+    ``query_temp`` = (coef, every): the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1).
+    ``borrows``: the layer has no keys and values of its own (no tensors for 'k', 'v' and what belongs to them); its runs
+    read the cache entry that another layer's run wrote, which has the same kv heads and sizes.
     ``score_softcap`` c: a scaled score s enters the softmax as c tanh(s / c).
     Without 'v' the values are the keys as projected (with their bias, before norm and rotation): value_dim
     must equal key_dim."""
@@ -262,7 +267,8 @@ class GeneralAttention(Mixer):
                  value_dim: int, position: Optional[PositionEncoding], scale: float, mask_chunk: Optional[int] = None,
                  mask_window: Optional[int] = None, mask_keep_first: int = 0, norm_eps: float = 0.0,
                  unit_norm_after_rotation: bool = False, score_softcap: Optional[float] = None, conv_taps: int = 0,
-                 value_position: Optional[PositionEncoding] = None):
+                 value_position: Optional[PositionEncoding] = None, norm_rows: bool = False,
+                 query_temp: Optional[Tuple[float, int]] = None, borrows: bool = False):
         if num_heads % num_kv_heads:
             raise ValueError(f"attention: {num_heads} heads are not a multiple of {num_kv_heads} kv heads")
         if unit_norm_after_rotation and (names.get("q_norm") or names.get("k_norm")):
@@ -285,7 +291,22 @@ class GeneralAttention(Mixer):
         self.softcap = float(score_softcap) if score_softcap is not None else 0.0
         self.taps = int(conv_taps)
         self.names = dict(names)
-        self.values_are_keys = "v" not in self.names
+        self.borrows, self.norm_rows = bool(borrows), bool(norm_rows)
+        self.values_are_keys = "v" not in self.names and not self.borrows
+        self.temp_coef, self.temp_every = (float(query_temp[0]), int(query_temp[1])) if query_temp is not None else (0.0, 0)
+        if query_temp is not None and self.temp_every <= 0:
+            raise ValueError(f"attention: a query temperature that grows every {query_temp[1]} positions")
+        if self.borrows and (any(self.names.get(k) for k in ("k", "v", "k_bias", "v_bias", "k_norm", "k_conv", "v_conv"))
+                             or conv_taps or unit_norm_after_rotation or self.names.get("gate")):
+            raise ValueError("attention: a layer that borrows keys and values has no tensors for them")
+        if self.norm_rows and (not self.names.get("q_norm") or bool(self.names.get("k_norm")) == self.borrows or conv_taps
+                               or self.values_are_keys or unit_norm_after_rotation or value_position is not None
+                               or any(self.names.get(k) for k in ("q_bias", "k_bias", "v_bias", "temp", "gate"))):
+            raise ValueError("attention: a norm over whole projections goes with q_norm and k_norm, and with no biases, "
+                             "convolution, values that are keys, number a head on the scores, gate a feature or rotated values")
+        if self.norm_rows and max(num_heads * key_dim, num_kv_heads * value_dim) > ops.QKV_ROW_MAX:
+            raise ValueError(f"attention: a projection of {max(num_heads * key_dim, num_kv_heads * value_dim)} features is "
+                             f"more than the kernel that norms it holds ({ops.QKV_ROW_MAX})")
         if self.taps and (self.values_are_keys or self.names.get("gate") or self.names.get("head_gate")):
             raise ValueError("attention: the convolution goes with q, k and v of their own and no output gate")
         if self.names.get("gate") and (self.names.get("head_gate") or value_position is not None):
@@ -300,9 +321,11 @@ class GeneralAttention(Mixer):
         self.hidden_size, self.nh, self.nkv, self.dk, self.dv = hidden_size, num_heads, num_kv_heads, key_dim, value_dim
         self.position, self.scale, self.chunk = position, float(scale), int(mask_chunk or 0)
         self.window, self.keep_first, self.norm_eps = int(mask_window or 0), int(mask_keep_first), float(norm_eps)
-        stacked = [(self.names["q"], num_heads * key_dim), (self.names["k"], num_kv_heads * key_dim)]
-        biases = [self.names.get("q_bias"), self.names.get("k_bias")]
-        if not self.values_are_keys:
+        stacked, biases = [(self.names["q"], num_heads * key_dim)], [self.names.get("q_bias")]
+        if not self.borrows:
+            stacked.append((self.names["k"], num_kv_heads * key_dim))
+            biases.append(self.names.get("k_bias"))
+        if not self.values_are_keys and not self.borrows:
             stacked.append((self.names["v"], num_kv_heads * value_dim))
             biases.append(self.names.get("v_bias"))
         self.norm_after = bool(unit_norm_after_rotation)
@@ -321,7 +344,8 @@ class GeneralAttention(Mixer):
                         bias_names=[self.names["out_bias"]] if self.names.get("out_bias") else None)
         # what the plain rotate-and-store kernel does not do
         self._extras = bool(any(biases) or self.names.get("q_norm") or self.names.get("k_norm") or self.values_are_keys
-                            or self.norm_after or self.taps or self.names.get("temp") or value_position is not None)
+                            or self.norm_after or self.taps or self.names.get("temp") or value_position is not None
+                            or self.temp_every)
         self.conv_widths = (num_heads * key_dim, num_kv_heads * key_dim, num_kv_heads * value_dim)
 
     def parts(self) -> List[Part]:
@@ -329,7 +353,8 @@ class GeneralAttention(Mixer):
 
     def weight_specs(self):
         from .base import WeightSpec
-        specs = [WeightSpec(self.names[k], (self.dk,), "norm") for k in ("q_norm", "k_norm") if self.names.get(k)]
+        specs = [WeightSpec(self.names[k], (self.dk * (heads if self.norm_rows else 1),), "norm")
+                 for k, heads in (("q_norm", self.nh), ("k_norm", self.nkv)) if self.names.get(k)]
         if self.names.get("sink"):
             specs.append(WeightSpec(self.names["sink"], (self.nh,), "small"))
         if self.names.get("temp"):
@@ -373,6 +398,8 @@ class GeneralAttention(Mixer):
             raise ValueError(f"attention: the rotation covers {rd} features, a head has {dk}")
         if self.taps and not writes_cache:
             raise ValueError("attention: a run that reads another run's cache has no convolution state of its own")
+        if self.borrows and writes_cache:
+            raise ValueError("attention: a layer that borrows keys and values has none to write")
         gated = self.gate_off is not None or self.head_gate_off is not None
         v_freq = None
         if self.value_position is not None:
@@ -380,7 +407,8 @@ class GeneralAttention(Mixer):
             if 2 * v_freq.shape[0] != dv:
                 raise ValueError(f"attention: the values' rotation covers {2 * v_freq.shape[0]} features, a value has {dv}")
         with ctx.timed("attn_qkv_rope"):
-            qkv = self.qkv.forward(h, ctx, "attn.qkv", rows=None if (writes_cache or gated) else nh * dk)
+            qkv = self.qkv.forward(h, ctx, "attn.qkv", rows=None if (writes_cache or gated) else nh * dk,
+                                   partials=self.norm_rows)
             if self.taps:
                 # the projected rows mixed over time, in float; the slot's state moves on to the step's last rows
                 mixed = ctx.ws.get("attn.conv", (n, sum(self.conv_widths)), torch.float32)
@@ -388,13 +416,22 @@ class GeneralAttention(Mixer):
                               max(ctx.q_lens), update_state=True, activation=False)
                 qkv = mixed
             q = ctx.ws.get("attn.q", (n, nh * dk), self.rt.dtype)
-            if self._extras:
+            head_gate = None
+            if self.norm_rows:
+                if self.head_gate_off is not None:
+                    head_gate = ctx.ws.get("attn.head_gate", (n, nh), self.rt.dtype)
+                ops.qkv_row_norm_store(qkv, q, nh, nkv, dk, dv, rd, ctx.positions, ctx.tok_slot, inv_freq, mag,
+                                       cache.streams["k"], cache.streams["v"], cache.page_table, cache.page_size, self.q_norm,
+                                       self.k_norm, self.norm_eps, write_kv=writes_cache, temp_coef=self.temp_coef,
+                                       temp_every=self.temp_every, interleaved=self.interleaved,
+                                       gate_col=self.head_gate_off or 0, gate_out=head_gate)
+            elif self._extras:
                 ops.qkv_norm_rotate_store(qkv, q, nh, nkv, dk, dv, rd, ctx.positions, ctx.tok_slot, inv_freq, mag,
                                           cache.streams["k"], cache.streams["v"], cache.page_table, cache.page_size,
                                           write_kv=writes_cache, bias=self.qkv.bias, q_norm=self.q_norm,
                                           k_norm=self.k_norm, eps=self.norm_eps, values_from_keys=self.values_are_keys,
                                           norm_after=self.norm_after, interleaved=self.interleaved, q_scale=self.temp,
-                                          v_inv_freq=v_freq)
+                                          v_inv_freq=v_freq, temp_coef=self.temp_coef, temp_every=self.temp_every)
             else:
                 ops.qkv_rotate_store(qkv, q, nh, nkv, dk, dv, rd, ctx.positions, ctx.tok_slot, inv_freq, mag,
                                      cache.streams["k"], cache.streams["v"], cache.page_table, cache.page_size,
@@ -405,7 +442,8 @@ class GeneralAttention(Mixer):
         gate = qkv[:, self.gate_off:self.gate_off + nh * dv] if self.gate_off is not None else None
         fin = None
         if finish:
-            head_gate = qkv[:, self.head_gate_off:self.head_gate_off + nh] if self.head_gate_off is not None else None
+            if self.head_gate_off is not None and head_gate is None:
+                head_gate = qkv[:, self.head_gate_off:self.head_gate_off + nh]
             fin = ops.HeadFinish(ctx.ws.get("attn.out", (n, nh * dv), self.rt.dtype), v_freq, head_gate, self.interleaved)
         with ctx.timed("attn_core"):
             # the matrix-core kernel (and the merge of split keys) applies the gate as it writes; the merge also turns

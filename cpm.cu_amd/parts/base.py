@@ -207,12 +207,14 @@ class ReplacingBranch:
 
 class StreamsBranch:
     """A sub-layer's result that joins a residual of several streams (hyper-connections): all streams at once,
-    x_t <- sum_s ``mix``[s, t] x_s + ``out``[t] * ``branch`` (mix float32 [S, S] indexed [from, to], out float32
-    [S]).  ``branch`` is a tensor [n, H], float partial sums [P, n, H] or a BiasedBranch.  It is left pending like
+    x_t <- sum_s ``mix``[s, t] x_s + ``out``[t] * ``scale`` * ``branch`` (mix float32 [S, S] indexed [from, to], out
+    float32 [S]).  ``branch`` is a tensor [n, H], float partial sums [P, n, H] or a BiasedBranch.  It is left pending like
     every branch and added by the norm that follows (``Norm.forward_streams``)."""
 
-    def __init__(self, branch, mix: torch.Tensor, out: torch.Tensor):
-        self.branch, self.mix, self.out = branch, mix, out
+    def __init__(self, branch, mix: torch.Tensor, out: torch.Tensor, scale: float = 1.0):
+        self.branch, self.mix, self.out, self.scale = branch, mix, out, float(scale)
+        if isinstance(branch, BiasedBranch) and self.scale != 1.0:
+            self.branch = branch.evaluate()             # the kernel scales the branch before its bias joins
 
     def pieces(self):
         """(tensor, bias or None) of the branch."""

@@ -283,14 +283,16 @@ class HyperConnectionBlock(Block):
     """Pre-norm sub-layers over a residual of S streams (hyper-connections).  Sub-layer q (1: mixer, 2:
     feed-forward, which a layer may lack) has numbers in[S], out[S] and mix[S, S] of its own:
 
-        u = sum_s in[s] x_s;   y = sub(norm(u));   x_t <- sum_s mix[s, t] x_s + out[t] * y    (all t at once)
+        u = sum_s in[s] x_s;   y = sub(norm(u));   x_t <- sum_s mix[s, t] x_s + m out[t] * y    (all t at once)
+
+    with m = ``residual_scale``.
 
     The result is left pending as a StreamsBranch and added by the norm that follows, which reads the streams with
     the next sub-layer's ``in`` in the same pass (Norm.forward_streams).
     ``names``: for each sub-layer the checkpoint tensors (in, out, mix)."""
 
     def __init__(self, mixer_norm: Norm, mixer: Mixer, streams: int, names: List[tuple], ff_norm: Optional[Norm] = None,
-                 feed_forward: Optional[FeedForward] = None):
+                 feed_forward: Optional[FeedForward] = None, residual_scale: float = 1.0):
         if (feed_forward is None) != (ff_norm is None):
             raise ValueError("hyper_connections: a feed-forward comes with its norm, or neither is given")
         if len(names) != (2 if feed_forward is not None else 1):
@@ -299,6 +301,7 @@ class HyperConnectionBlock(Block):
             raise ValueError(f"hyper_connections: {streams} streams")
         self.mixer_norm, self.mixer, self.ff_norm, self.feed_forward = mixer_norm, mixer, ff_norm, feed_forward
         self.streams, self.names = int(streams), [tuple(t) for t in names]
+        self.residual_scale = float(residual_scale)
 
     def parts(self) -> List[Part]:
         return [self.mixer_norm, self.mixer] + ([self.ff_norm, self.feed_forward] if self.feed_forward is not None else [])
@@ -321,12 +324,12 @@ class HyperConnectionBlock(Block):
         with ctx.timed("attn"):
             with ctx.timed("norm"):
                 h = self.mixer_norm.forward_streams(x, stream.take_pending(), read, ctx, tag="block.h")
-            pending = StreamsBranch(self.mixer.forward(h, ctx, cache, writes_cache), mix, out)
+            pending = StreamsBranch(self.mixer.forward(h, ctx, cache, writes_cache), mix, out, self.residual_scale)
         if self.feed_forward is not None:
             read, out, mix = self.numbers[1]
             with ctx.timed("ffn"):
                 with ctx.timed("norm"):
                     h = self.ff_norm.forward_streams(x, pending, read, ctx, tag="block.h")
-                pending = StreamsBranch(self.feed_forward.forward(h, ctx), mix, out)
+                pending = StreamsBranch(self.feed_forward.forward(h, ctx), mix, out, self.residual_scale)
         stream.pending = pending
         stream.pending_scale = 1.0

@@ -1,4 +1,4 @@
-"""Gated feed-forward: down( act(x Wg^T) * (x Wu^T) ), act = SiLU (or the tanh form of GELU, or a clamped swish).
+"""Feed-forwards: gated, down( act(x Wg^T) * (x Wu^T) ), act = SiLU (or the tanh form of GELU, or a clamped swish).
 
 gate and up are one stacked product, gate rows first (src/model/ffn.cuh:31-59,
 77-84); silu(g) * u in float (src/model/activation.cuh:6-18).
@@ -52,6 +52,29 @@ class GatedFFN(FeedForward):
             return self.down.forward(act, ctx, "ffn.down", out_dtype=torch.float32, partials=True)
 
 
+@FEED_FORWARDS.register("plain")
+class PlainFFN(FeedForward):
+    """down( act(up x) ) without a gate; act is 'silu', 'gelu_tanh' or 'relu_squared' (max(z, 0)^2)."""
+
+    def __init__(self, up_name: str, down_name: str, hidden_size: int, intermediate_size: int, activation: str):
+        try:
+            self.activation = ops.plain_activation(activation)
+        except ops.KernelError as e:
+            raise ValueError(f"feed-forward: {e}") from None
+        self.hidden_size, self.intermediate_size = hidden_size, intermediate_size
+        self.up = Linear([(up_name, intermediate_size)], hidden_size)
+        self.down = Linear([(down_name, hidden_size)], intermediate_size)
+
+    def parts(self) -> List[Part]:
+        return [self.up, self.down]
+
+    def forward(self, h: torch.Tensor, ctx: StepContext):
+        with ctx.timed("ffn_up"):
+            act = self.up.forward_activated(h, ctx, "ffn.up", self.activation)
+        with ctx.timed("ffn_down"):
+            return self.down.forward(act, ctx, "ffn.down", out_dtype=torch.float32, partials=True)
+
+
 @FEED_FORWARDS.register("poly_norm")
 class PolyNormFFN(FeedForward):
     """down( act(up x) ) with the PolyNorm activation act(z) = a N(z) + b N(z^2) + c N(z^3) + e: powers element by
@@ -89,17 +112,19 @@ class PolyNormFFN(FeedForward):
 
 @FEED_FORWARDS.register("routed_experts")
 class RoutedExpertsFFN(FeedForward):
-    """A mixture of small gated feed-forwards (no biases), of which every token uses ``top``.
+    """A mixture of small feed-forwards (gated unless said otherwise, no biases), of which every token uses ``top``.
 
     Router: logits z = W_router h in float, scores s = softmax(z) over all experts (``score`` 'sigmoid': sigmoid of
-    every logit alone).  The choice goes by s + a correction a expert (a checkpoint tensor; the weights use s without
+    every logit alone; with 'router_bias' in ``names`` a number an expert is added to the logits first).  The choice goes by s + a correction a expert (a checkpoint tensor; the weights use s without
     it).  With ``groups`` = (count, keep) the experts form ``count`` equal groups of neighbours, a group's score is
     its largest choice score (``group_score`` 'top2_sum': the sum of its two largest), and only experts of the
     ``keep`` best groups can be chosen.  The chosen experts' outputs are added with weights s / (sum of the chosen s +
     1e-20) * ``weight_scale``.  A shared expert (``shared_size``) runs for every token and is added, times
     sigmoid(w . h), one number a token, if ``names`` holds 'shared_scale'.  ``activation`` / ``shared_activation``:
     the experts' and the shared expert's nonlinearity as GatedFFN takes it.  Without ``normalize`` the weights are
-    s * ``weight_scale``.  ``identity``: so many further rows of the router (and of the correction) are identity
+    s * ``weight_scale``.  ``score`` 'logit': the choice goes by z itself (+ the correction) and the weights are the
+    softmax of the chosen experts' z among themselves.  Without ``gated`` an expert is down(act(up h)) with
+    ``activation`` as PlainFFN takes it (the shared expert stays gated).  ``identity``: so many further rows of the router (and of the correction) are identity
     experts, which have no tensors and give the layer's input back.
 
     ``names``: 'router', 'correction' (or absent), 'expert' (a format with {e} for the expert's number and {part}
@@ -108,7 +133,7 @@ class RoutedExpertsFFN(FeedForward):
     def __init__(self, names: Mapping[str, str], hidden_size: int, expert_size: int, experts: int, top: int,
                  groups: Optional[Tuple[int, int]] = None, shared_size: Optional[int] = None, score: str = "softmax",
                  group_score: str = "max", weight_scale: float = 1.0, activation="silu", shared_activation=None,
-                 normalize: bool = True, identity: int = 0):
+                 normalize: bool = True, identity: int = 0, gated: bool = True):
         routes = experts + identity
         if experts < 1 or identity < 0 or routes > ops.MOE_MAX_EXPERTS:
             raise ValueError(f"routed_experts: {experts} experts and {identity} identity experts (one to "
@@ -122,8 +147,13 @@ class RoutedExpertsFFN(FeedForward):
         if score not in ops.MOE_SCORES or group_score not in ops.MOE_GROUP_SCORES:
             raise ValueError(f"routed_experts: score '{score}' ({sorted(ops.MOE_SCORES)}) or group score "
                              f"'{group_score}' ({sorted(ops.MOE_GROUP_SCORES)})")
+        if score == "logit" and not normalize:
+            raise ValueError("routed_experts: weights that are a softmax of the chosen logits are normalised")
+        if not gated and shared_size is not None and shared_activation is None:
+            raise ValueError("routed_experts: the shared expert is gated and needs a nonlinearity of its own")
+        self.gated = bool(gated)
         try:
-            self.activation = ops.gate_activation(activation)
+            self.activation = ops.gate_activation(activation) if self.gated else ops.plain_activation(activation)
         except ops.KernelError as e:
             raise ValueError(f"routed_experts: {e}") from None
         self.score, self.group_score, self.weight_scale = score, group_score, float(weight_scale)
@@ -139,6 +169,9 @@ class RoutedExpertsFFN(FeedForward):
                                    activation=shared_activation if shared_activation is not None else activation)
         self.shared_gated = self.shared is not None and bool(self.names.get("shared_scale"))
 
+    def _in_parts(self) -> Tuple[str, ...]:
+        return ("gate", "up") if self.gated else ("up",)
+
     def _expert(self, e: int, part: str) -> str:
         return self.names["expert"].format(e=e, part=part)
 
@@ -150,9 +183,11 @@ class RoutedExpertsFFN(FeedForward):
         specs = [WeightSpec(self.names["router"], (self.routes, H))]
         if self.names.get("correction"):
             specs.append(WeightSpec(self.names["correction"], (self.routes,), "slight"))
+        if self.names.get("router_bias"):
+            specs.append(WeightSpec(self.names["router_bias"], (self.routes,), "small"))
         for e in range(self.experts):
-            specs += [WeightSpec(self._expert(e, "gate"), (F, H)), WeightSpec(self._expert(e, "up"), (F, H)),
-                      WeightSpec(self._expert(e, "down"), (H, F))]
+            specs += [WeightSpec(self._expert(e, part), (F, H)) for part in self._in_parts()]
+            specs.append(WeightSpec(self._expert(e, "down"), (H, F)))
         if self.shared_gated:
             specs.append(WeightSpec(self.names["shared_scale"], (1, H)))
         return specs
@@ -162,6 +197,7 @@ class RoutedExpertsFFN(FeedForward):
         f32 = lambda name: tensors[name].to(torch.float32).contiguous()
         self.router = f32(self.names["router"])
         self.correction = f32(self.names["correction"]) if self.names.get("correction") else None
+        self.router_bias = f32(self.names["router_bias"]) if self.names.get("router_bias") else None
         self.shared_scale = f32(self.names["shared_scale"]).reshape(-1) if self.shared_gated else None
         # steps of many tokens: the router as a product of the library's, bf16 operands summed in float.  A bf16 weight
         # times a bf16 row is exact in float, so this is the float product of the kernel for few tokens
@@ -170,8 +206,8 @@ class RoutedExpertsFFN(FeedForward):
         if rt.dtype == torch.bfloat16 and all(t.dtype == torch.bfloat16 for t in named):
             last = named[1].reshape(1, -1) if self.shared_gated else torch.zeros_like(named[0][:1])
             self.router_rows = torch.cat([named[0], last]).contiguous()       # [routes + 1, H], as the logits lie
-        # an expert's gate rows, then its up rows: [E, 2F, H]; down: [E, H, F]
-        self.gate_up = torch.stack([torch.cat([tensors[self._expert(e, "gate")], tensors[self._expert(e, "up")]], 0)
+        # an expert's gate rows, then its up rows: [E, 2F, H] (without a gate [E, F, H]); down: [E, H, F]
+        self.gate_up = torch.stack([torch.cat([tensors[self._expert(e, part)] for part in self._in_parts()], 0)
                                     for e in range(self.experts)]).to(rt.dtype).contiguous()
         self.down = torch.stack([tensors[self._expert(e, "down")] for e in range(self.experts)]).to(rt.dtype).contiguous()
 
@@ -192,7 +228,8 @@ class RoutedExpertsFFN(FeedForward):
                 torch.mm(h, self.router_rows.t(), out_dtype=torch.float32, out=logits)
             ops.moe_route(h, self.router, self.correction, self.shared_scale, self.groups[0], self.groups[1], self.top,
                           idx, wts, sg, logits, score=self.score, group_score=self.group_score,
-                          weight_scale=self.weight_scale, normalize=self.normalize, logits_ready=many)
+                          weight_scale=self.weight_scale, normalize=self.normalize, logits_ready=many,
+                          bias=self.router_bias)
         shared = self.shared.forward(h, ctx) if self.shared is not None else None
         act = ctx.ws.get("moe.act", (n, self.top, self.expert_size), self.rt.dtype)
         out = ctx.ws.get("moe.out", (n, self.hidden_size), torch.float32) if join is None else None
@@ -208,9 +245,12 @@ class RoutedExpertsFFN(FeedForward):
                 tile_expert = ctx.ws.get("moe.tile_expert", (tiles,), torch.int32)
                 n_tiles = ctx.ws.get("moe.n_tiles", (1,), torch.int32)
                 ops.moe_experts_mfma(h, self.gate_up, self.down, idx, wts, out, act, y, rows, tile_expert, n_tiles,
-                                     shared, sg, activation=self.activation, join=join)
+                                     shared, sg, activation=self.activation, join=join, gated=self.gated)
             else:
                 # few tokens: an expert's weights stream once for every token that chose it
-                ops.moe_gated(h, self.gate_up, idx, act, activation=self.activation)
+                if self.gated:
+                    ops.moe_gated(h, self.gate_up, idx, act, activation=self.activation)
+                else:
+                    ops.moe_up(h, self.gate_up, idx, act, self.activation)
                 ops.moe_down(act, self.down, idx, wts, out, shared, sg, h=h, join=join)
         return out

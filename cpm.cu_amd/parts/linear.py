@@ -81,6 +81,17 @@ class Linear(Part):
         ops.linear(x, w, out, alpha, w_tiled=wt)
         return out
 
+    def forward_activated(self, x: torch.Tensor, ctx: StepContext, tag: str, activation: str) -> torch.Tensor:
+        """act(x W^T), [n, out] of x's type, for a feed-forward without a gate (ops.plain_activation)."""
+        n = x.shape[0]
+        act = ctx.ws.get(tag + ".act", (n, self.out_features), x.dtype)
+        if ops.skinny_ok(x):
+            ops.gemm_skinny(x, self.tiled if self.tiled is not None else self.weight, act, mode="act", activation=activation)
+        else:
+            ops.linear(x, self.weight, act)
+            ops.activate(act, activation)
+        return act
+
     def forward_float(self, x: torch.Tensor, ctx: StepContext, tag: str) -> torch.Tensor:
         """x [n, in] -> float32 [n, out], or float partial sums [S, n, out], whatever the number of rows: for a result
         that takes the place of the residual, which is never rounded to 16 bits."""

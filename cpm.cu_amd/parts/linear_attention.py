@@ -1,4 +1,7 @@
-"""Linear attention with a fixed decay a head: a recurrence whose state is a matrix a head and which has neither a
+"""Linear attention with a fixed decay a head (DecayLinearAttention), or with a learned decay a head and key channel
+(GatedLinearAttention, below).
+
+The first is a recurrence whose state is a matrix a head and which has neither a
 softmax nor a denominator,
 
     S <- d_h S + k v^T;   o = S^T q          S: [dim, vdim], zero at the start; d_h a constant of the configuration
@@ -103,3 +106,95 @@ class DecayLinearAttention(Mixer):
                                 gate_after="silu" if self.gate_activation == "silu" else True)
         with ctx.timed("linattn_out"):
             return self.out_proj.forward(gated, ctx, "linattn.out", out_dtype=torch.float32, partials=True)
+
+
+@MIXERS.register("gated_linear_attention")
+class GatedLinearAttention(Mixer):
+    """Linear attention whose decay is a number a head and key channel, made from the token by a low-rank product:
+
+        S <- diag(a) S + k v^T;   o = S^T q                       S: [dim, vdim] a head, zero at the start
+        a = sigmoid(W_up (W_down h) + b)^(1/tau),   q = W_q h * query_scale
+
+    Each head's o is divided by its root mean square (eps inside the root), multiplied by a weight of vdim numbers
+    shared by the heads and by silu(gate) (``gate_activation`` 'sigmoid': sigmoid(gate)), then projected out.  One input
+    projection gives [q | k | v | gate | W_down h]; everything behind it runs in float, and S lives as float fixed-size
+    state in the sequence's cache slot.  A step of one token a sequence is one kernel between the two projections."""
+
+    def __init__(self, names: Mapping[str, str], hidden_size: int, heads: int, key_dim: int, value_dim: int,
+                 decay_rank: int, tau: float, eps: float, query_scale: Optional[float] = None,
+                 gate_activation: str = "silu"):
+        """``names``: checkpoint tensors for 'q', 'k', 'v', 'gate', 'out', 'norm', 'decay_down', 'decay_up', 'decay_bias'.
+        ``query_scale``: dim^(-1/2) if not given."""
+        if key_dim > 256:
+            raise ValueError(f"gated_linear_attention: a key size of {key_dim} is not supported (at most 256)")
+        if decay_rank < 1 or not tau > 0:
+            raise ValueError(f"gated_linear_attention: a decay of rank {decay_rank} with tau {tau}")
+        if gate_activation not in ("silu", "sigmoid"):
+            raise ValueError(f"gated_linear_attention: gate nonlinearity '{gate_activation}' (silu or sigmoid)")
+        self.names = dict(names)
+        self.hidden_size, self.heads, self.dk, self.dv = hidden_size, heads, key_dim, value_dim
+        self.rank, self.tau, self.eps, self.gate_activation = int(decay_rank), float(tau), float(eps), gate_activation
+        self.query_scale = float(query_scale) if query_scale is not None else key_dim ** -0.5
+        n, hk, hv = self.names, heads * key_dim, heads * value_dim
+        self.in_proj = Linear([(n["q"], hk), (n["k"], hk), (n["v"], hv), (n["gate"], hv), (n["decay_down"], self.rank)],
+                              hidden_size)
+        self.out_proj = Linear([(n["out"], hidden_size)], hv)
+        self.g_off, self.low_off = 2 * hk + hv, 2 * hk + 2 * hv
+
+    def parts(self) -> List[Part]:
+        return [self.in_proj, self.out_proj]
+
+    def weight_specs(self) -> List[WeightSpec]:
+        n, hk = self.names, self.heads * self.dk
+        return [WeightSpec(n["decay_up"], (hk, self.rank)), WeightSpec(n["decay_bias"], (hk,), "small"),
+                WeightSpec(n["norm"], (self.dv,), "norm")]
+
+    def bind(self, tensors: Mapping[str, torch.Tensor], rt: Runtime):
+        f = lambda k: tensors[self.names[k]].to(torch.float32)
+        self.up_w, self.up_b = f("decay_up").t().contiguous(), f("decay_bias").contiguous()
+        self.norm_head = f("norm").contiguous()
+        self.norm_w = self.norm_head.repeat(self.heads).contiguous()
+        self.rt = rt
+
+    def cache_needs(self) -> CacheNeeds:
+        return CacheNeeds(state=(("memory", StateSpec((self.heads, self.dv, self.dk), torch.float32)),))
+
+    def reserve_workspace(self, ws, rt: Runtime, max_step_tokens: int, max_slots: int):
+        rows = ops.gla_segment_rows(max_step_tokens, self.heads, self.dv)
+        if rows:
+            ws.get("gla.seg_state", (rows, self.heads, self.dv, self.dk), torch.float32)
+            ws.get("gla.seg_decay", (rows, self.heads, self.dk), torch.float32)
+
+    def forward(self, h: torch.Tensor, ctx: StepContext, cache: Optional[CacheView], writes_cache: bool = True):
+        if not writes_cache:
+            raise ValueError("gated_linear_attention: a run that reads another run's cache has no state of its own")
+        n, hk, hv = h.shape[0], self.heads * self.dk, self.heads * self.dv
+        with ctx.timed("linattn_in"):
+            u = self.in_proj.forward(h, ctx, "gla.in")
+        gated = ctx.ws.get("gla.gated", (n, hv), self.rt.dtype)
+        state = cache.state["memory"]
+        if ctx.single_token:
+            with ctx.timed("linattn_scan"):
+                ops.gla_step(u, 0, hk, 2 * hk, self.g_off, self.low_off, self.up_w, self.up_b, self.tau, self.norm_head, self.eps,
+                             state, gated, ctx.cu_q, ctx.seq_slot, self.heads, self.dk, self.dv, self.query_scale,
+                             self.gate_activation)
+        else:
+            decay = ctx.ws.get("gla.decay", (n, hk), torch.float32)
+            y = ctx.ws.get("gla.y", (n, hv), torch.float32)
+            with ctx.timed("linattn_prepare"):
+                ops.channel_decay(u[:, self.low_off:self.low_off + self.rank], self.up_w, self.up_b, self.tau, decay)
+            segments, seg_len = ops.gla_segments(ctx.q_lens, self.heads, self.dv)
+            scratch = None
+            if segments > 1:
+                rows = len(ctx.q_lens) * segments
+                scratch = (ctx.ws.get("gla.seg_state", (rows, self.heads, self.dv, self.dk), torch.float32),
+                           ctx.ws.get("gla.seg_decay", (rows, self.heads, self.dk), torch.float32),
+                           ctx.ws.get("gla.qa", (n, hk), torch.float32))
+            with ctx.timed("linattn_scan"):
+                ops.gla_scan(u, 0, hk, 2 * hk, decay, state, y, ctx.cu_q, ctx.seq_slot, self.heads, self.dk, self.dv,
+                             self.query_scale, segments, seg_len, scratch)
+            with ctx.timed("linattn_norm"):
+                ops.rms_norm_groups(y, self.norm_w, self.eps, gated, groups=self.heads, gate=u[:, self.g_off:self.g_off + hv],
+                                    gate_after="silu" if self.gate_activation == "silu" else True)
+        with ctx.timed("linattn_out"):
+            return self.out_proj.forward(gated, ctx, "gla.out", out_dtype=torch.float32, partials=True)

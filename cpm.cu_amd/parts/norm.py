@@ -91,9 +91,10 @@ def _streams_norm(norm, x, pending: Optional[StreamsBranch], read, ctx: StepCont
     n_out = x.shape[-2] if rows is None else rows.shape[0]
     out = ctx.ws.get(tag, (n_out, norm.hidden_size), norm.rt.dtype)
     branch = bias = mix = outw = None
+    scale = 1.0
     if pending is not None:
-        (branch, bias), mix, outw = pending.pieces(), pending.mix, pending.out
-    ops.streams_norm(x, branch, bias, 1.0, mix, outw, read, norm.weight, norm.eps, out, rows, rms=rms)
+        (branch, bias), mix, outw, scale = pending.pieces(), pending.mix, pending.out, pending.scale
+    ops.streams_norm(x, branch, bias, scale, mix, outw, read, norm.weight, norm.eps, out, rows, rms=rms)
     return out
 
 
