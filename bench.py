@@ -172,7 +172,7 @@ def main():
     ap.add_argument("--perf", action="store_true",
                     help="after the timed runs, a few eager steps with the engine's timers on: average ms by kernel "
                          "class (products / attention / selection / norms / head) on stderr and under 'timers'")
-    ap.add_argument("--scenario", default="headline", choices=["headline", "small_batch64", "sparse32k", "duvulix", "gumodra", "sagedra", "nelutar", "pemalorn"],
+    ap.add_argument("--scenario", default="headline", choices=["headline", "small_batch64", "sparse32k", "duvulix", "gumodra", "sagedra", "nelutar", "pemalorn", "tirizen"],
                     help="headline: the 8B shape at batch 8, context 4,096 (the default line); "
                          "small_batch64: the 0.5B shape, 64 unequal prompts through the generation loop; sparse32k: "
                          "the 8B shape with InfLLM-v2 at 32k context; duvulix: four Duvulix layers of a real model's "
@@ -186,7 +186,10 @@ def main():
                          "channel, retention, routed experts, a layer that runs twice) beside the four Sagedra layers; pemalorn: four Pemalorn layer "
                          "runs of a real model's sizes (latent attention under a window, attention with rotated values "
                          "twice, routed and identity experts, input convolutions, a token table) beside the four Duvulix "
-                         "and the four Gumodra layers")
+                         "and the four Gumodra layers; tirizen: four Tirizen layers of a real model's sizes (gated linear "
+                         "attention, attention with norms over whole projections, a layer that reads another's keys, "
+                         "feed-forwards and experts without a gate, four residual streams) beside the four Nelutar and "
+                         "the four Sagedra layers")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py: this engine runs on one GPU; --gpus {args.gpus} is not supported (no multi-GPU path exists)")
@@ -674,6 +677,55 @@ def pemalorn_step_bytes(raw, esize, batch, context, prefill=False):
     return weights * esize + batch * per_seq, int(weights)
 
 
+def config_tirizen():
+    """Four layers of sizes that resemble a real model's: width 4,096 in 4 residual streams; gated linear attention of 32
+    heads of 128 by 128 (decays of rank 16), attention with 32 heads on 8 kv heads of 128, and a layer of the same attention
+    that reads the other's keys and values; a feed-forward of 16,512 without a gate (as many numbers as a gated one of
+    11,008) and 64 experts of 2,112 (gated: 1,408), 6 a token."""
+    gla = {"heads": 32, "dim": 128, "vdim": 128, "tau": 16.0}
+    attn = {"heads": 32, "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "q_temp": {"coef": 0.1, "every": 1024}}
+    moe = {"kind": "moe", "expert": {"ff": 2112}, "router": {"experts": 64, "top": 6}}
+    return {
+        "architecture": "Tirizen", "vocab": 73448, "width": 4096, "norm": {"eps": 1e-6}, "embedding": {"scale": 64.0},
+        "max_positions": 8192, "residual_mult": 0.7, "streams": 4, "logit_scale": 0.25,
+        "layers": [
+            {"type": "gla", "mixer": dict(gla), "mlp": {"kind": "dense", "ff": 16512}},
+            {"type": "attention", "mixer": dict(attn), "mlp": moe},
+            {"type": "gla", "mixer": dict(gla), "mlp": moe},
+            {"type": "attention", "mixer": dict(attn, kv_from=1), "mlp": moe},
+        ],
+    }
+
+
+def tirizen_step_bytes(raw, esize, batch, context, prefill=False):
+    """Bytes a decode step must move: every matrix that the step reads once (of a mixture: the router, and an expert for
+    every (token, choice) pair, at most all of them), and per sequence what the mixers read: keys and values (a layer that
+    borrows them reads them again), the recurrent states read and written, the row of the position table.  With
+    ``prefill``: the matrix elements a prompt token is multiplied with (of a mixture: the chosen experts only)."""
+    W = raw["width"]
+    weights = raw["vocab"] * W
+    per_seq = W * esize
+    for layer in raw["layers"]:
+        m = layer["mixer"]
+        if layer["type"] == "gla":
+            hk, hv = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+            weights += (2 * hk + 3 * hv + 16) * W + 16 * hk
+            per_seq += 2 * 4 * m["heads"] * m["dim"] * m["vdim"]
+        else:
+            weights += m["heads"] * (m["dim"] + m["vdim"] + 1) * W
+            if m.get("kv_from") is None:
+                weights += m["kv_heads"] * (m["dim"] + m["vdim"]) * W
+            per_seq += context * m["kv_heads"] * (m["dim"] + m["vdim"]) * esize
+        mlp = layer["mlp"]
+        if mlp["kind"] == "dense":
+            weights += 2 * mlp["ff"] * W
+        else:
+            r = mlp["router"]
+            pairs = r["top"] if prefill else min(max(batch, 1) * r["top"], r["experts"])
+            weights += r["experts"] * W + pairs * 2 * mlp["expert"]["ff"] * W
+    return weights * esize + batch * per_seq, weights
+
+
 def duvulix_scenario(args, dev):
     """Decode and prefill of the Duvulix layer shapes beside the MiniCPM4-8B layer shape (equal width, equal
     number of layers, random weights): one JSON line with both models' figures and their timers by kernel class."""
@@ -704,6 +756,14 @@ def pemalorn_scenario(args, dev):
     (parallel layers with a softmax sink and routed experts): equal width, vocabulary and number of layer runs."""
     layer_shapes_scenario(args, dev, "pemalorn", "Pemalorn", config_pemalorn(), ("duvulix", config_duvulix()),
                           ("gumodra", config_gumodra()))
+
+
+def tirizen_scenario(args, dev):
+    """The same for the Tirizen layer shapes beside the Nelutar (linear attention with decays, routed experts) and the
+    Sagedra layer shapes (a residual of four streams, a matrix-state recurrence): equal width, vocabulary, number of layers,
+    and numbers a feed-forward."""
+    layer_shapes_scenario(args, dev, "tirizen", "Tirizen", config_tirizen(), ("nelutar", config_nelutar()),
+                          ("sagedra", config_sagedra()))
 
 
 def layer_shapes_scenario(args, dev, first, title, first_raw, *others):
@@ -789,6 +849,10 @@ def layer_shapes_scenario(args, dev, first, title, first_raw, *others):
             step_bytes = lambda b: pemalorn_step_bytes(raw, esize, b, args.context)[0]
             params = pemalorn_step_bytes(raw, esize, args.batch, 0)[1]
             prefill_params = pemalorn_step_bytes(raw, esize, 1, 0, prefill=True)[1]
+        elif name == "tirizen":
+            step_bytes = lambda b: tirizen_step_bytes(raw, esize, b, args.context)[0]
+            params = tirizen_step_bytes(raw, esize, args.batch, 0)[1]
+            prefill_params = tirizen_step_bytes(raw, esize, 1, 0, prefill=True)[1]
         else:
             step_bytes = lambda b: weight_bytes_per_step(cfg, esize) + b * args.context * kv_bytes_per_token(cfg, esize)
             params = weight_bytes_per_step(cfg, esize) // esize
@@ -853,6 +917,9 @@ def other_scenarios(args, dev):
         return
     if args.scenario == "pemalorn":
         pemalorn_scenario(args, dev)
+        return
+    if args.scenario == "tirizen":
+        tirizen_scenario(args, dev)
         return
     import torch
     from cpmcu_amd import Engine, EngineOptions, StepEntry

@@ -15,6 +15,7 @@
 //
 // Keys and values lie in their pages as common.h says (key_index, value_index), each with its own head size.
 #include "common.h"
+#include "vec4.h"
 
 enum { DST_ROWS = 0, DST_KEYS = 1, DST_VALUES = 2 };
 
@@ -837,7 +838,7 @@ __global__ __launch_bounds__(1024) void qkv_row_norm_store_kernel(
     int temp_every, const int* __restrict__ positions, const int* __restrict__ tok_slot, const float* __restrict__ inv_freq,
     float mag, T* __restrict__ kpool, T* __restrict__ vpool, PagedView pv, int pool_hdk, int pool_hdv, int interleaved,
     long gate_col, T* __restrict__ gate_out) {
-    extern __shared__ float row_s[];
+    extern __shared__ __attribute__((aligned(16))) float row_s[];
     __shared__ float red[17];
     const long t = blockIdx.x;
     const int what = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
@@ -851,11 +852,13 @@ __global__ __launch_bounds__(1024) void qkv_row_norm_store_kernel(
         return v;
     };
     float ss = 0.f;
-    if (nparts <= 1) {
-        for (int i = threadIdx.x; i < width; i += blockDim.x) {
-            const float v = to_f32(src[i]);
-            row_s[i] = v;
-            ss += v * v;
+    const bool vec = (ld & 3) == 0 && (part_stride & 3) == 0 && (nh * dk) % 4 == 0 && (nkv * dk) % 4 == 0 && width % 4 == 0 &&
+                     (uintptr_t)qkv % 16 == 0;
+    if (vec) {
+        for (int i = 4 * threadIdx.x; i < width; i += 4 * blockDim.x) {
+            const float4 v = nparts == 1 ? load4(src + i) : sum_parts4(src + i, nparts, part_stride);
+            *(float4*)(row_s + i) = v;
+            ss += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
         }
     } else {
         for (int i = threadIdx.x; i < width; i += blockDim.x) {
@@ -885,10 +888,21 @@ __global__ __launch_bounds__(1024) void qkv_row_norm_store_kernel(
     float r = 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps);
     if (what == 0 && temp_every > 0) r *= 1.0f + temp_coef * logf((float)((pos + 1) / temp_every) + 1.0f);
     const float* nw_ = what == 0 ? q_norm_w : k_norm_w;
-    // (each thread finishes the values it wrote itself)
+    const long prow = what == 1 ? paged_row(pv, tok_slot[t], pos) : 0;
+    if (vec && rot_dims == 0 && dk % 4 == 0 && (uintptr_t)q_out % 16 == 0) {
+        // four features a thread, straight to where they belong (each thread finishes the values it wrote itself)
+        const int d4 = dk / 4;
+        for (int j = threadIdx.x; j < width / 4; j += blockDim.x) {
+            const float4 v = *(const float4*)(row_s + 4 * j), w = *(const float4*)(nw_ + 4 * j);
+            const int h = j / d4, d = 4 * (j - h * d4);
+            T* dst = what == 0 ? q_out + t * width + 4 * j : kpool + key_index(prow, h, nkv, pool_hdk) + key_d_offset(d);
+            store4(dst, v.x * r * w.x, v.y * r * w.y, v.z * r * w.z, v.w * r * w.w);
+        }
+        return;
+    }
+    __syncthreads();
     for (int i = threadIdx.x; i < width; i += blockDim.x) row_s[i] *= r * nw_[i];
     __syncthreads();
-    const long prow = what == 1 ? paged_row(pv, tok_slot[t], pos) : 0;
     for (int h = wave; h < heads; h += nw) {
         const float* s = row_s + (long)h * dk;
         if (what == 0) rotate_run(s, q_out + (t * nh + h) * dk, dk, rot_dims, pos, inv_freq, mag, DST_ROWS, 0, lane, 64, interleaved);
@@ -922,7 +936,7 @@ extern "C" const char* cpmcu_qkv_row_norm_store(const void* qkv, int in_dtype, l
     PagedView pv{page_table, table_width, page_size};
     // few tokens: a row over many threads
     int block = 256;
-    while (n < 256 && block < 1024 && block * 2 <= width) block *= 2;
+    while (n < 256 && block < 1024 && block * 4 < width) block *= 2;
     const dim3 grid(n, write_kv ? 3 : 1);
 #define LAUNCH(ITv, Tv)                                                                                                \
     qkv_row_norm_store_kernel<ITv, Tv><<<grid, block, width * 4, stream>>>(                                            \

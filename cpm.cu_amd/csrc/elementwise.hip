@@ -26,12 +26,41 @@ __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict_
     }
 }
 
+// the same with four columns a thread (H a multiple of 4, aligned rows)
+template <typename T>
+__global__ void embed_vec4_kernel(const T* __restrict__ table, const int* __restrict__ ids, float* __restrict__ out,
+                                  int H, float scale, const T* __restrict__ pos_table, const int* __restrict__ positions,
+                                  int copies, long copy_stride) {
+    const long r = blockIdx.x;
+    const T* src = table + (long)ids[r] * H;
+    const T* add = pos_table ? pos_table + (long)positions[r] * H : nullptr;
+    float* dst = out + r * H;
+    for (int c = 4 * threadIdx.x; c < H; c += 4 * blockDim.x) {
+        const float4 v = load4(src + c);
+        const float4 a = add ? load4(add + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+        const float4 o = make_float4(v.x * scale + a.x, v.y * scale + a.y, v.z * scale + a.z, v.w * scale + a.w);
+        for (int s = 0; s < copies; ++s) *(float4*)(dst + s * copy_stride + c) = o;
+    }
+}
+
 extern "C" const char* cpmcu_embed(const void* table, int dtype, const int* ids, float* out, int n, int H, int V,
                                    float scale, const void* pos_table, const int* positions, int copies,
                                    hipStream_t stream) {
     CPMCU_REQUIRE(n > 0 && H > 0 && V > 0 && copies > 0, "embed: empty shape n=%d H=%d V=%d copies=%d", n, H, V, copies);
     CPMCU_REQUIRE(!pos_table || positions, "embed: a table of positions without positions");
     CPMCU_REQUIRE(dtype == CPMCU_F32 || dtype == CPMCU_BF16, "embed: unknown dtype %d", dtype);
+    if (H % 4 == 0 && (uintptr_t)table % 16 == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)pos_table % 16 == 0) {
+        int vblock = 64;
+        while (vblock < (n >= 512 ? 256 : 1024) && vblock * 4 < H) vblock *= 2;
+        if (dtype == CPMCU_F32)
+            embed_vec4_kernel<float><<<n, vblock, 0, stream>>>((const float*)table, ids, out, H, scale, (const float*)pos_table,
+                                                              positions, copies, (long)n * H);
+        else
+            embed_vec4_kernel<bf16_t><<<n, vblock, 0, stream>>>((const bf16_t*)table, ids, out, H, scale, (const bf16_t*)pos_table,
+                                                               positions, copies, (long)n * H);
+        CPMCU_LAUNCH_CHECK("embed");
+        return nullptr;
+    }
     const int block = H >= 1024 ? 256 : 64;
     if (dtype == CPMCU_F32)
         embed_kernel<float><<<n, block, 0, stream>>>((const float*)table, ids, out, H, scale, (const float*)pos_table, positions,

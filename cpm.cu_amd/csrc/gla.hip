@@ -248,7 +248,22 @@ __global__ __launch_bounds__(256) void gla_fix_kernel(const float* __restrict__ 
             acc[u] = gfloatx4_t{0.f, 0.f, 0.f, 0.f};
             qp[u] = qa + (long)(first + min(t0 + u * 16 + r, n_q - 1)) * heads * dk + (long)h * dk;
         }
-        for (int n0 = 0; n0 < dk; n0 += 4) {
+        int n0 = 0;
+        if (dk % 4 == 0)                             // 16 features at a time: a lane brings 4 neighbouring ones of its rows
+            for (; n0 + 16 <= dk; n0 += 16) {
+                const float4 s = *(const float4*)(sp + n0 + 4 * g);
+                float4 q[TB];
+#pragma unroll
+                for (int u = 0; u < TB; ++u) q[u] = *(const float4*)(qp[u] + n0 + 4 * g);
+#pragma unroll
+                for (int u = 0; u < TB; ++u) {
+                    acc[u] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[u].x, s.x, acc[u], 0, 0, 0);
+                    acc[u] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[u].y, s.y, acc[u], 0, 0, 0);
+                    acc[u] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[u].z, s.z, acc[u], 0, 0, 0);
+                    acc[u] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[u].w, s.w, acc[u], 0, 0, 0);
+                }
+            }
+        for (; n0 < dk; n0 += 4) {
             const int n = min(n0 + g, dk - 1);
             const float s = n0 + g < dk ? sp[n] : 0.f;
 #pragma unroll

@@ -275,7 +275,8 @@ def test_whole_row_norms_into_the_cache(dtype, shape, parts):
     q2, g2 = torch.empty_like(q_out), torch.empty_like(gates)
     ops.qkv_row_norm_store(borrowed, q2, H, G, d, dv, rd, pos, slot, freq, 1.0, None, None, None, page, dev(qn), None, eps, write_kv=False,
                            temp_coef=coef, temp_every=every, gate_col=H * d, gate_out=g2)
-    assert torch.equal(q2, q_out) and torch.equal(g2, gates) and torch.equal(kp, before[0]) and torch.equal(vp, before[1])
+    close(q2, q.reshape(T, H * d), dtype, what="queries without keys")
+    assert torch.equal(g2, gates) and torch.equal(kp, before[0]) and torch.equal(vp, before[1])
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
