@@ -1,4 +1,4 @@
-"""cpm.cu_amd: a small generation engine (MiniCPM4, Duvulix, Gumodra, Sagedra, Nelutar, Pemalorn) for one AMD MI355X (gfx950).
+"""cpm.cu_amd: a small generation engine (MiniCPM4, Duvulix, Gumodra, Sagedra, Nelutar, Pemalorn, Tirizen) for one AMD MI355X (gfx950).
 
 Importable as ``cpmcu_amd`` (the folder name ``cpm.cu_amd`` is not a Python
 identifier; ``cpmcu_amd`` beside it is a link to the same folder).

@@ -294,6 +294,30 @@ def test_ranks_come_from_the_checkpoint(models, tmp_path, dtype, rank):
     assert again.model.layers[1].mixer.rank == rank
 
 
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("kinds", ["g", "a", "gg", "aa"])
+def test_models_of_one_kind_of_layer(tmp_path, dtype, kinds):
+    """No layer with pages, or none with a state; in the last one the second layer has no keys of its own and no layer a
+    feed-forward."""
+    from cpmcu_amd import Engine, EngineOptions
+    raw = dict(tt.tiny_d(), streams=4, residual_mult=0.5)
+    att = {"heads": 4, "kv_heads": 2, "dim": 24, "vdim": 12, "scale": 0.3, "q_temp": {"coef": 0.5, "every": 16}}
+    layers = [{"type": "gla", "mixer": {"heads": 3, "dim": 24, "vdim": 20, "tau": 6.0}, "mlp": {"kind": "dense", "ff": 56}} if k == "g"
+              else {"type": "attention", "mixer": dict(att, **({"kv_from": 0} if i else {})), "mlp": None} for i, k in enumerate(kinds)]
+    raw["layers"] = layers
+    d = str(tmp_path / "m")
+    tt.write_model(raw, d, 541)
+    cfg, w = read(d)
+    reqs = {"a": tiny.random_tokens(140, raw["vocab"], 6200), "b": tiny.random_tokens(66, raw["vocab"], 6201), "c": tiny.random_tokens(1, raw["vocab"], 6202)}
+    refs = {r: Reference(cfg, w, t, conditioning=True) for r, t in reqs.items()}
+    eng = Engine.from_dir(d, EngineOptions(dtype=dtype, max_tokens=512, max_slots=3, hip_graph=True))
+    assert eng.cache.has_state == ("g" in kinds)
+    check(schedules.tail(eng, reqs, 70), refs, dtype, kinds)
+    check(schedules.batched(eng, reqs, {"a": 100, "b": 60, "c": 1}, [("b", "a", "c")]), refs, dtype, kinds + " batched")
+    eng.cache.check()
+    assert not eng.cache.live
+
+
 def test_sequences_longer_than_the_position_table_are_refused(models):
     from cpmcu_amd import Engine, EngineOptions, StepEntry
     d, cfg, w, reqs, _ = models["D"]

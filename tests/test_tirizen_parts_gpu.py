@@ -84,7 +84,7 @@ def test_streams_with_a_scaled_branch(S, H, n):
 # ---------------------------------------------------------------------------
 # gated linear attention
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("n, R, C, tau", [(1, 1, 5, 16.0), (9, 16, 96, 16.0), (30, 70, 300, 1.0), (17, 130, 257, 3.5)])
+@pytest.mark.parametrize("n, R, C, tau", [(1, 1, 5, 12.0), (9, 12, 84, 6.0), (30, 70, 300, 1.0), (17, 130, 257, 3.5)])
 def test_decays_a_channel(dtype, n, R, C, tau):
     """Among them decays next to zero and next to one, which keep their relative precision, and that of 1 - a."""
     from cpmcu_amd import ops
@@ -123,7 +123,7 @@ def _gla_inputs(T, H, dk, dv, dtype, g, R=5):
     return rows, offs, up, b, ops_, at("g", hv)
 
 
-SHAPES = [(2, 48, 32), (3, 20, 36), (5, 13, 7), (1, 200, 1), (2, 128, 48), (1, 256, 33), (4, 8, 24), (2, 70, 130), (1, 64, 64), (2, 33, 16)]
+SHAPES = [(3, 44, 28), (3, 20, 36), (5, 13, 7), (1, 200, 1), (2, 128, 48), (1, 256, 33), (4, 8, 24), (2, 70, 130), (1, 64, 64), (2, 33, 16)]
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
@@ -280,7 +280,7 @@ def test_whole_row_norms_into_the_cache(dtype, shape, parts):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("H, G, d, dv", [(6, 2, 24, 40), (4, 4, 96, 96), (8, 1, 128, 128)])
+@pytest.mark.parametrize("H, G, d, dv", [(6, 2, 24, 40), (4, 4, 80, 80), (8, 1, 128, 128)])
 def test_far_keys_and_gated_heads(dtype, H, G, d, dv):
     """Over pages in disorder, whole prompts and single tokens (whole and split keys): for chosen queries one key's score
     stands far above the rest, at position 0, at both sides of page borders, far back, among hundreds alike; each head
@@ -383,7 +383,7 @@ def test_router_with_a_bias(dtype, score, n, H, E, top):
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("n, H, F, E, top", [(3, 96, 40, 6, 3), (1, 100, 20, 2, 1), (9, 64, 16, 64, 6), (130, 64, 24, 4, 2), (200, 128, 264, 3, 3),
-                                             (70, 96, 30, 8, 8), (5, 512, 256, 12, 1), (600, 256, 96, 16, 4)])
+                                             (70, 96, 30, 8, 8), (5, 512, 256, 12, 1), (600, 192, 72, 12, 3)])
 def test_experts_without_a_gate(dtype, n, H, F, E, top):
     """The products for few tokens and, bfloat16, the grouped ones."""
     from cpmcu_amd import ops
